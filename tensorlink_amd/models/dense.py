@@ -463,4 +463,7 @@ def _stage_class(config: ModelConfig):
     if config.architecture == "potosun":
         from tensorlink_amd.models.potosun import PotosunStageModel
         return PotosunStageModel
+    if config.architecture == "mogisun":
+        from tensorlink_amd.models.mogisun import MogisunStageModel
+        return MogisunStageModel
     return StageModel

@@ -28,7 +28,8 @@ import torch.nn as nn
 
 from tensorlink_amd.models.configs import ModelConfig
 from tensorlink_amd.models.dense import TLLinear
-from tensorlink_amd.models.layered import LayeredStage, load_named_tensors
+from tensorlink_amd.models.layered import (LayeredStage, load_named_tensors,
+                                           looped_runs, read_loop)
 from tensorlink_amd.models.mixers import (CanonConv, ConvSinkAttention,
                                           LayerNormWeight, ParallelMixer,
                                           PolyNormFF, SSDMixer)
@@ -73,13 +74,8 @@ class DizepelConfig(ModelConfig):
                     (right["heads"] * right["vdim"]) % right["norm_groups"]:
                 raise KeyError(f"layer {i}: heads / groups / norm_groups of "
                                "the state-space mixer do not divide")
-        loop = cfg.get("loop") or {}
         n = len(layers)
-        start, stop = int(loop.get("start", 0)), int(loop.get("stop", 0))
-        times = int(loop.get("times", 0)) if loop else 0
-        if loop and not (0 <= start <= stop <= n and times >= 1):
-            raise KeyError("loop: need 0 <= start <= stop <= layers and "
-                           "times >= 1")
+        start, stop, times = read_loop(cfg, n)
         heads = max(lc["mixer"]["left"]["heads"] for lc in layers)
         kvh = max(lc["mixer"]["left"]["kv_heads"] for lc in layers)
         dim = max(lc["mixer"]["left"]["dim"] for lc in layers)
@@ -98,13 +94,8 @@ class DizepelConfig(ModelConfig):
     def layer_runs(self) -> List[Tuple[int, Optional[int]]]:
         """(layer index, pass number or None) in execution order; every
         run has its own cache entry."""
-        n = len(self.layer_specs)
-        if not self.loop_times:
-            return [(i, None) for i in range(n)]
-        runs = [(i, None) for i in range(self.loop_start)]
-        for t in range(self.loop_times):
-            runs += [(i, t) for i in range(self.loop_start, self.loop_stop)]
-        return runs + [(i, None) for i in range(self.loop_stop, n)]
+        return looped_runs(len(self.layer_specs), self.loop_start,
+                           self.loop_stop, self.loop_times)
 
     def param_count(self, include_embeddings: bool = True) -> int:
         w = self.hidden_size

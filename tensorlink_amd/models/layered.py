@@ -13,7 +13,7 @@ usual stage interface (embed / forward / head / make_kv_cache).
 from __future__ import annotations
 
 import os
-from typing import Dict, Iterable, Tuple
+from typing import Dict, Iterable, List, Optional, Tuple
 
 import torch
 import torch.nn as nn
@@ -70,6 +70,32 @@ class LayeredStage(nn.Module):
         return self.embed_tokens(input_ids)
 
 
+def looped_runs(n: int, start: int, stop: int,
+                times: int) -> List[Tuple[int, Optional[int]]]:
+    """(layer index, pass number or None) of ``n`` layers in execution
+    order when layers start .. stop-1 run ``times`` times in a row with the
+    same weights (times 0: no looped span). Every run has its own cache
+    entry."""
+    if not times:
+        return [(i, None) for i in range(n)]
+    runs = [(i, None) for i in range(start)]
+    for t in range(times):
+        runs += [(i, t) for i in range(start, stop)]
+    return runs + [(i, None) for i in range(stop, n)]
+
+
+def read_loop(cfg: dict, n: int) -> Tuple[int, int, int]:
+    """(start, stop, times) of config.json's optional ``loop`` over ``n``
+    layers; times 0 without one."""
+    loop = cfg.get("loop") or {}
+    start, stop = int(loop.get("start", 0)), int(loop.get("stop", 0))
+    times = int(loop.get("times", 0))
+    if loop and not (0 <= start <= stop <= n and times >= 1):
+        raise KeyError("loop: need 0 <= start <= stop <= layers and "
+                       "times >= 1")
+    return start, stop, times
+
+
 def tensor_shapes(ckpt_dir: str) -> Dict[str, Tuple[int, ...]]:
     """Tensor name -> shape from the header of ``model.safetensors`` in
     ``ckpt_dir`` (an 8-byte little-endian length, then that many bytes of
@@ -93,7 +119,8 @@ def load_named_tensors(params: Dict[str, torch.Tensor],
                        partial: Dict[str, int] = None) -> int:
     """Fill ``params`` from ``model.safetensors``. ``names`` maps a
     checkpoint tensor to (parameter, row offset — or expert index for a
-    stacked 3-d parameter). Strict both ways: an unknown tensor raises and
+    stacked 3-d parameter, optionally followed by the row offset inside the
+    expert's matrix). Strict both ways: an unknown tensor raises and
     so does a parameter left (partly) unfilled, unless listed in
     ``optional`` and untouched; ``partial`` names parameters that the
     checkpoint fills only up to the given number of elements (the rest
@@ -106,13 +133,14 @@ def load_named_tensors(params: Dict[str, torch.Tensor],
         for key in f.keys():
             if key not in names:
                 raise KeyError(f"unexpected tensor {key!r} in checkpoint")
-            pname, off = names[key]
+            pname, off = names[key][:2]
             t = f.get_tensor(key)
             p = params[pname]
+            if p.dim() == 3:                        # stacked experts
+                p, off = p[off], (names[key][2] if len(names[key]) > 2
+                                  else 0)
             if p.dim() == 0:
                 p.copy_(t.reshape(()))
-            elif p.dim() == 3:                      # stacked experts
-                p[off].copy_(t)
             else:
                 if t.shape[1:] != p.shape[1:] or off + t.shape[0] > p.shape[0]:
                     raise KeyError(f"tensor {key!r} has shape "

@@ -142,6 +142,11 @@ def load_stage_from_checkpoint(stage: StageModel, ckpt_dir: str,
         n = load_potosun_weights(stage, ckpt_dir, dtype=dtype)
         stage.to(device=device, dtype=dtype)
         return n
+    if arch == "mogisun":
+        from tensorlink_amd.models.mogisun import load_mogisun_weights
+        n = load_mogisun_weights(stage, ckpt_dir, dtype=dtype)
+        stage.to(device=device, dtype=dtype)
+        return n
     from safetensors import safe_open
 
     index_path = os.path.join(ckpt_dir, "model.safetensors.index.json")
@@ -196,6 +201,10 @@ def init_random_stage(stage: StageModel, device="cpu", dtype=torch.bfloat16,
     if stage.config.architecture == "potosun":
         from tensorlink_amd.models.potosun import init_potosun_random
         init_potosun_random(stage, seed=seed)
+        return stage.to(device=device, dtype=dtype)
+    if stage.config.architecture == "mogisun":
+        from tensorlink_amd.models.mogisun import init_mogisun_random
+        init_mogisun_random(stage, seed=seed)
         return stage.to(device=device, dtype=dtype)
     gen_dev = device if str(device).startswith("cuda") else "cpu"
     g = torch.Generator(device=gen_dev)

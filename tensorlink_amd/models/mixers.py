@@ -242,6 +242,12 @@ class GroupLimitedMoE(nn.Module, _F32Cache):
 # attention, latent attention, windowed attention with score mixing and a
 # sink, plain two-matrix feed-forward, per-layer token input
 # ---------------------------------------------------------------------------
+def pad_cols(n: int) -> int:
+    """Rows of a fused projection rounded up to what the serving GEMM
+    kernels take (a multiple of 64); the added rows are zero."""
+    return (n + 63) // 64 * 64
+
+
 class RMSWeight(nn.Module, _F32Cache):
     """Weight of an RMS norm; ``one_plus`` = stored around zero and
     applied as (1 + w)."""
@@ -417,6 +423,16 @@ class WindowAttention(nn.Module, _F32Cache):
     ``out_gate``     the concatenated heads times sigmoid of one more
                      projection of the input (``g`` rows of the fused
                      projection);
+    ``unit_norm``    the query / key norm is per head without a weight
+                     (instead of ``qk_norm``'s weights);
+    ``q_temp``       (coef, every): the query at position p is multiplied by
+                     1 + coef ln(floor((p + 1) / every) + 1);
+    ``head_gate``    head h's output times sigmoid of one more projection of
+                     the input (``g`` rows, one per head);
+    ``bias``         the q, k, v and output projections have biases;
+    ``side_cols``    this many further rows of the fused projection, with a
+                     bias, belong to the caller: forward then returns
+                     (output, projection, their first column);
     ``v_mix``        value mixing across layers: the first such layer of a
                      model publishes its values of the step's tokens in the
                      ``shared`` dictionary handed to forward, later ones
@@ -434,10 +450,14 @@ class WindowAttention(nn.Module, _F32Cache):
                  chunk: int = 0, keep_first: int = 0,
                  sink_logits: bool = False, rel_rows: int = 0,
                  rel_far: float = 0.0, out_gate: bool = False,
-                 v_mix: bool = False):
+                 v_mix: bool = False, unit_norm: bool = False,
+                 q_temp: Optional[tuple] = None, head_gate: bool = False,
+                 bias: bool = False, side_cols: int = 0):
         super().__init__()
         assert heads % kv_heads == 0 and rot_dims % 2 == 0 and rot_dims <= dim
         assert not (chunk and window), "a chunked mask has no window"
+        assert not (unit_norm and qk_norm) and not (head_gate and out_gate)
+        assert bias or not side_cols, "the caller's rows have a bias"
         self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
         self.scale, self.eps = float(scale), float(eps)
         self.rot_dims, self.base = int(rot_dims), rot_base
@@ -448,9 +468,15 @@ class WindowAttention(nn.Module, _F32Cache):
         self.v_mix = bool(v_mix)
         self.q_cols, self.k_cols = heads * dim, kv_heads * dim
         self.v_cols = kv_heads * vdim
-        self.g_cols = heads * vdim if out_gate else 0
-        self.qkv = TLLinear(width, self.q_cols + self.k_cols + self.v_cols
-                            + self.g_cols, bias=False)
+        self.unit_norm, self.head_gate = bool(unit_norm), bool(head_gate)
+        self.q_temp = tuple(float(x) for x in q_temp) if q_temp else None
+        self.side_cols = int(side_cols)
+        self.side_col = self.q_cols + self.k_cols + self.v_cols
+        self.g_col = self.side_col + self.side_cols
+        self.g_cols = heads if head_gate else heads * vdim if out_gate else 0
+        cols = self.g_col + self.g_cols
+        self.qkv = TLLinear(width, pad_cols(cols) if side_cols else cols,
+                            bias=bias)
         self.q_norm = nn.Parameter(torch.ones(
             dim if head_norm else self.q_cols)) if qk_norm else None
         self.k_norm = nn.Parameter(torch.ones(
@@ -463,7 +489,7 @@ class WindowAttention(nn.Module, _F32Cache):
         self.vmix = nn.Parameter(torch.zeros(())) if v_mix else None
         if rel_rows:
             self.buckets = mx.log_distance_buckets(rel_rows, rel_far)
-        self.o_proj = TLLinear(heads * vdim, width, bias=False)
+        self.o_proj = TLLinear(heads * vdim, width, bias=bias)
 
     def cache_spec(self):
         return {"kind": "kv", "G": self.G, "DK": self.D, "V": self.V}
@@ -497,8 +523,8 @@ class WindowAttention(nn.Module, _F32Cache):
         kpool, vpool = cache.k[layer_idx], cache.v[layer_idx]
         v_col = self.q_cols + self.k_cols
         rot = dict(rot_dims=self.rot_dims, freqs=fr,
-                   interleaved=self.interleaved, head_norm=self.head_norm,
-                   eps=self.eps)
+                   interleaved=self.interleaved,
+                   head_norm=self.head_norm or self.unit_norm, eps=self.eps)
         mx.norm_rope_rows(proj, self.q_cols, self.G, self.D, meta,
                           norm_w=kn, norm_cols=self.k_cols, pool=kpool, **rot)
         first = None
@@ -519,7 +545,7 @@ class WindowAttention(nn.Module, _F32Cache):
                               mix_src=first[0], mix_col=first[1],
                               mix_lam=self._f32("vmix").reshape(1))
         q = mx.norm_rope_rows(proj, 0, self.H, self.D, meta, norm_w=qn,
-                              norm_cols=self.q_cols, **rot)
+                              norm_cols=self.q_cols, temp=self.q_temp, **rot)
         o = mx.flex_attention(
             q, kpool, vpool, meta, self.H, self.scale, window=self.window,
             sink=self.sink,
@@ -529,8 +555,10 @@ class WindowAttention(nn.Module, _F32Cache):
             chunk=self.chunk, keep_first=self.keep_first,
             dist_bias=self._dist_bias(h.device) if self.rel is not None
             else None,
-            gate=proj if self.g_cols else None,
-            gate_col=v_col + self.v_cols, out_dtype=h.dtype)
+            gate=proj if self.g_cols else None, gate_col=self.g_col,
+            gate_heads=self.head_gate, out_dtype=h.dtype)
+        if self.side_cols:
+            return self.o_proj(o), proj, self.side_col
         return self.o_proj(o)
 
 
@@ -548,17 +576,29 @@ class DenseFF(nn.Module):
 
 
 class GatedFF(nn.Module):
-    """down(gelu(gate x) * (up x)), tanh-form or exact GELU, no biases;
-    gate and up are one fused projection [gate | up]."""
+    """down(act(gate x) * (up x)), no biases; ``act`` is the tanh-form or
+    exact GELU (``tanh_form``) or "silu"; gate and up are one fused
+    projection [gate | up]. ``side_cols`` further rows of it, with a bias,
+    belong to the caller: forward then returns (output, projection, their
+    first column)."""
 
-    def __init__(self, width: int, ff: int, tanh_form: bool = True):
+    kind = "dense"
+
+    def __init__(self, width: int, ff: int, tanh_form: bool = True, *,
+                 act: Optional[str] = None, side_cols: int = 0):
         super().__init__()
-        self.ff, self.tanh_form = int(ff), bool(tanh_form)
-        self.gate_up = TLLinear(width, 2 * ff, bias=False)
+        self.ff, self.side_cols = int(ff), int(side_cols)
+        self.act = act or ("gelu_tanh" if tanh_form else "gelu")
+        self.side_col = 2 * self.ff
+        self.gate_up = TLLinear(
+            width, pad_cols(2 * ff + side_cols) if side_cols else 2 * ff,
+            bias=bool(side_cols))
         self.down = TLLinear(ff, width, bias=False)
 
     def forward(self, h):
-        return self.down(mx.gelu_gate(self.gate_up(h), self.tanh_form))
+        p = self.gate_up(h)
+        y = self.down(mx.act_gate(p, self.act, self.ff))
+        return (y, p, self.side_col) if self.side_cols else y
 
 
 class TokenSide(nn.Module):
@@ -762,3 +802,109 @@ class PolyNormFF(nn.Module, _F32Cache):
 
     def forward(self, h):
         return self.down(mx.polynorm(self.up(h), self._f32("act"), self.eps))
+
+
+# ---------------------------------------------------------------------------
+# blocks of the gated-residual family: gated linear attention with one decay
+# per key channel, mixture of gated experts with a shared expert
+# ---------------------------------------------------------------------------
+class GatedLinearAttention(nn.Module, _F32Cache):
+    """Linear attention whose memory decays per key channel and token:
+    S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t with
+    alpha = sigmoid(a2 (a1 x) + a2_b)^(1/tau), q scaled by dim^-1/2; every
+    head's read-out is RMS-normed over vdim with one shared weight, times
+    silu of a gate projection, then the output projection.
+
+    One fused projection [q | k | v | g | caller's ``side_cols`` | a1]; the
+    low-rank second factor a2 and everything behind it run in fp32 inside
+    the recurrence's kernels. With ``side_cols`` (rows with a bias) forward
+    returns (output, projection, their first column). Per-sequence memory:
+    the fp32 state [heads, dim, vdim]."""
+
+    kind = "gla"
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int,
+                 rank: int, tau: float, eps: float, *, side_cols: int = 0):
+        super().__init__()
+        self.H, self.D, self.V, self.R = heads, dim, vdim, int(rank)
+        self.tau, self.eps = float(tau), float(eps)
+        hd, hv = heads * dim, heads * vdim
+        self.offs = (0, hd, 2 * hd)                      # q | k | v
+        self.g_col = 2 * hd + hv
+        self.side_cols, self.side_col = int(side_cols), 2 * hd + 2 * hv
+        self.a_col = self.side_col + self.side_cols
+        self.proj = TLLinear(width, pad_cols(self.a_col + self.R),
+                             bias=bool(side_cols))
+        self.a2 = nn.Parameter(torch.zeros(hd, self.R))
+        self.a2_b = nn.Parameter(torch.zeros(hd))
+        self.norm = nn.Parameter(torch.ones(vdim))
+        self.o_proj = TLLinear(hv, width, bias=False)
+
+    def cache_spec(self):
+        return {"kind": "state", "shapes": [(self.H, self.D, self.V)]}
+
+    def _a2t(self):
+        """a2 transposed, fp32 [rank, heads*dim]; rebuilt when it changes."""
+        p = self.a2
+        key = (p.data_ptr(), p._version, p.device, p.dtype)
+        hit = self.__dict__.get("_a2t_hit")
+        if hit is None or hit[0] != key:
+            hit = (key, p.detach().float().t().contiguous())
+            self.__dict__["_a2t_hit"] = hit
+        return hit[1]
+
+    def forward(self, h, meta, cache, layer_idx, shared=None):
+        proj = self.proj(h)
+        (S,) = cache.state[layer_idx]
+        o = mx.gla_scan(proj, self.offs + (self.a_col,), self._a2t(),
+                        self._f32("a2_b"), self.tau, S, meta, self.H, self.D,
+                        self.V)
+        y = mx.rms_scale(o, self._f32("norm"), self.eps, False, gate=proj,
+                         gate_col=self.g_col, out_dtype=h.dtype,
+                         heads=self.H)
+        y = self.o_proj(y)
+        return (y, proj, self.side_col) if self.side_cols else y
+
+
+class GatedMoE(nn.Module, _F32Cache):
+    """Mixture of gated experts down(act(gate x) * (up x)), no biases:
+    fp32 router, the ``top`` largest logits chosen and weighted by the
+    softmax over the chosen ones; optionally a shared expert of the same
+    form (``shared_ff`` > 0) for every token, times sigmoid of one more
+    projection of the input.
+
+    The dense rows — the shared expert's gate and up, its sigmoid's row and
+    the caller's ``side_cols`` (with a bias) — are one fused projection
+    [gate | up | side | sg]; the routed experts are stacked and run as
+    grouped products over expert-sorted (token, choice) pairs."""
+
+    kind = "moe"
+
+    def __init__(self, width: int, ff: int, experts: int, top: int,
+                 shared_ff: int = 0, *, act: str = "silu",
+                 side_cols: int = 0):
+        super().__init__()
+        assert 1 <= top <= experts
+        self.W, self.ff, self.E, self.top = width, int(ff), experts, int(top)
+        self.sff, self.act = int(shared_ff), act
+        self.side_cols, self.side_col = int(side_cols), 2 * self.sff
+        self.sg_col = self.side_col + self.side_cols
+        self.router = nn.Parameter(torch.zeros(experts, width))
+        self.gate_up = nn.Parameter(torch.zeros(experts, 2 * self.ff, width))
+        self.down = nn.Parameter(torch.zeros(experts, width, self.ff))
+        cols = self.sg_col + (1 if self.sff else 0)
+        self.dense = TLLinear(width, pad_cols(cols), bias=bool(side_cols)) \
+            if cols else None
+        self.shared_down = TLLinear(self.sff, width, bias=False) \
+            if self.sff else None
+
+    def forward(self, h):
+        wts, idx = mx.topk_softmax_router(h, self._f32("router"), self.top)
+        p = self.dense(h) if self.dense is not None else None
+        s = (self.shared_down(mx.act_gate(p, self.act, self.sff))
+             if self.sff else None)
+        y = mx.expert_gated_ff(h, wts, idx, self.gate_up, self.down,
+                               self.act, shared=s,
+                               sgate=p if self.sff else None,
+                               sgate_col=self.sg_col)
+        return (y, p, self.side_col) if self.side_cols else y

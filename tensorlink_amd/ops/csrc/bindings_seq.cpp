@@ -19,14 +19,19 @@ void tl_rms_scale(const void* x, const void* w, const void* gate, int ldg,
                   int gate_col, void* out, int64_t rows, int N, float eps,
                   int one_plus, int is_f32, hipStream_t stream);
 void tl_add_rms(void* X, const void* y, const void* w, void* h, int64_t rows,
-                int W, float eps, float x_scale, int is_f32,
-                hipStream_t stream);
-void tl_gelu_gate(const void* p, void* out, int64_t rows, int N,
-                  int tanh_form, int is_f32, hipStream_t stream);
+                int W, float eps, float x_scale, const void* gate, int ldg,
+                int gate_aligned, int is_f32, hipStream_t stream);
+void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
+                 int64_t rows, int N, int act, int is_f32,
+                 hipStream_t stream);
+void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
+                      void* out, int64_t rows, int H, int V, float eps,
+                      int is_f32, hipStream_t stream);
 void tl_gelu(const void* x, void* out, int64_t n, int N, int tanh_form,
              const void* table, int ldt, int table_col, const void* tokens,
              int is_f32, hipStream_t stream);
-void tl_soft_cap(void* z, int64_t n, float cap, hipStream_t stream);
+void tl_soft_cap(void* z, int64_t n, float cap, float scale,
+                 hipStream_t stream);
 void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        int head_dim, const void* norm_w, int norm_cols,
                        float eps, int rot_off, int rot_dims,
@@ -35,6 +40,7 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        void* out, void* pool, int is_f32, int head_norm,
                        int interleaved, float rot_mult, const void* mix_src,
                        int mix_ld, int mix_col, const void* mix_lam,
+                       double temp_coef, double temp_every,
                        hipStream_t stream);
 int tl_flex_attn_heads_per_block(int H, int G, int DK, int V, int has_talk);
 int tl_flex_attn_rows(const void* q, const void* kpool, const void* vpool,
@@ -140,10 +146,11 @@ Tensor rms_scale(Tensor x, Tensor w, double eps, bool one_plus,
   return out;
 }
 
-// X (*= x_scale) += y; returns rms(X) * w in the serving dtype, or,
-// without a weight, X itself after the add
+// X (*= x_scale) += y [* sigmoid(gate columns)]; returns rms(X) * w in the
+// serving dtype, or, without a weight, X itself after the add
 Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
-               double eps, double x_scale, bool out_f32) {
+               double eps, double x_scale, c10::optional<Tensor> gate,
+               int64_t gate_col, bool out_f32) {
   SEQ_F32(X);
   TORCH_CHECK(X.dim() == 2, "X must be [T, W]");
   if (w.has_value()) {
@@ -156,6 +163,18 @@ Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
     TORCH_CHECK(act_is_f32(y.value()) == (out_f32 ? 1 : 0),
                 "y / output dtype mismatch");
   }
+  const char* gp = nullptr;
+  int ldg = 0, gate_aligned = 0;
+  if (gate.has_value()) {
+    SEQ_IN(gate.value());
+    TORCH_CHECK(y.has_value() && gate->scalar_type() == y->scalar_type() &&
+                    gate->dim() == 2 && gate->size(0) == X.size(0) &&
+                    gate_col >= 0 && gate_col + X.size(1) <= gate->size(1),
+                "gate must be [T, >= gate_col + W] of y's dtype");
+    ldg = (int)gate->size(1);
+    gp = (const char*)gate->data_ptr() + gate_col * gate->element_size();
+    gate_aligned = ldg % 4 == 0 && gate_col % 4 == 0;
+  }
   Tensor h = X;
   if (w.has_value())
     h = torch::empty(X.sizes(), X.options().dtype(out_f32 ? torch::kFloat
@@ -163,18 +182,51 @@ Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
   tl_add_rms(X.data_ptr(), y.has_value() ? y->data_ptr() : nullptr,
              w.has_value() ? w->data_ptr() : nullptr,
              w.has_value() ? h.data_ptr() : nullptr, X.size(0), (int)X.size(1),
-             (float)eps, (float)x_scale, out_f32 ? 1 : 0, seq_stream());
+             (float)eps, (float)x_scale, gp, ldg, gate_aligned,
+             out_f32 ? 1 : 0, seq_stream());
   return h;
 }
 
-// gelu(p[:, :N]) * p[:, N:] for p [T, 2N]
-Tensor gelu_gate(Tensor p, bool tanh_form) {
+// act(p[:, col:col + N]) * p[:, col + N:col + 2N]
+Tensor act_gate(Tensor p, int64_t col, int64_t N, int64_t act) {
   SEQ_IN(p);
-  TORCH_CHECK(p.dim() == 2 && p.size(1) % 2 == 0, "p must be [T, 2N]");
-  const int64_t N = p.size(1) / 2;
+  TORCH_CHECK(p.dim() == 2 && col >= 0 && N >= 1 &&
+                  col + 2 * N <= p.size(1) && act >= 0 && act <= 2,
+              "p must hold 2N columns from col");
   auto out = torch::empty({p.size(0), N}, p.options());
-  tl_gelu_gate(p.data_ptr(), out.data_ptr(), p.size(0), (int)N,
-               tanh_form ? 1 : 0, act_is_f32(p), seq_stream());
+  tl_act_gate((const char*)p.data_ptr() + col * p.element_size(), p.size(1),
+              p.size(1) % 8 == 0 && col % 8 == 0, out.data_ptr(), p.size(0),
+              (int)N, (int)act, act_is_f32(p), seq_stream());
+  return out;
+}
+
+// per head: x_h / rms(x_h) * w [* silu(gate columns)], x fp32 [T, H*V]
+Tensor head_rms_gate(Tensor x, Tensor w, int64_t H, double eps,
+                     c10::optional<Tensor> gate, int64_t gate_col,
+                     bool out_f32) {
+  SEQ_F32(x);
+  SEQ_F32(w);
+  const int64_t V = w.numel();
+  TORCH_CHECK(x.dim() == 2 && H >= 1 && x.size(1) == H * V,
+              "x must be [T, H * V], w [V]");
+  const char* gp = nullptr;
+  int ldg = 0;
+  if (gate.has_value()) {
+    SEQ_IN(gate.value());
+    TORCH_CHECK(act_is_f32(gate.value()) == (out_f32 ? 1 : 0),
+                "gate / output dtype mismatch");
+    TORCH_CHECK(gate->dim() == 2 && gate->size(0) == x.size(0) &&
+                    gate_col >= 0 && gate_col + H * V <= gate->size(1),
+                "gate columns out of range");
+    ldg = (int)gate->size(1);
+    gp = (const char*)gate->data_ptr() + gate_col * gate->element_size();
+  }
+  auto out = torch::empty(
+      x.sizes(),
+      x.options().dtype(out_f32 ? torch::kFloat : torch::kBFloat16));
+  tl_head_rms_gate(x.data_ptr(), w.data_ptr(), gp, ldg, out.data_ptr(),
+                   x.size(0), (int)H, (int)V, (float)eps, out_f32 ? 1 : 0,
+                   seq_stream());
   return out;
 }
 
@@ -204,9 +256,10 @@ Tensor gelu_mul(Tensor x, bool tanh_form, c10::optional<Tensor> table,
   return out;
 }
 
-void soft_cap_(Tensor z, double cap) {
+void soft_cap_(Tensor z, double cap, double scale) {
   SEQ_F32(z);
-  tl_soft_cap(z.data_ptr(), z.numel(), (float)cap, seq_stream());
+  tl_soft_cap(z.data_ptr(), z.numel(), (float)cap, (float)scale,
+              seq_stream());
 }
 
 void norm_rope_rows(Tensor src, int64_t col, int64_t n_heads,
@@ -217,7 +270,8 @@ void norm_rope_rows(Tensor src, int64_t col, int64_t n_heads,
                     c10::optional<Tensor> out, c10::optional<Tensor> pool,
                     bool head_norm, bool interleaved, double rot_mult,
                     c10::optional<Tensor> mix_src, int64_t mix_col,
-                    c10::optional<Tensor> mix_lam) {
+                    c10::optional<Tensor> mix_lam, double temp_coef,
+                    double temp_every) {
   SEQ_IN(src);
   SEQ_I32(tok_seq);
   SEQ_I32(tok_pos);
@@ -228,10 +282,13 @@ void norm_rope_rows(Tensor src, int64_t col, int64_t n_heads,
   TORCH_CHECK(col >= 0 && col + N <= ld, "columns out of range");
   TORCH_CHECK(tok_seq.numel() == T && tok_pos.numel() == T,
               "ragged metadata");
-  if (norm_w.has_value() && head_norm) {
-    SEQ_F32(norm_w.value());
-    TORCH_CHECK(norm_w->numel() == head_dim && n_heads <= 512,
-                "a per-head norm has one weight [head_dim] (<= 512 heads)");
+  if (head_norm) {
+    TORCH_CHECK(n_heads <= 512, "a per-head norm serves <= 512 heads");
+    if (norm_w.has_value()) {
+      SEQ_F32(norm_w.value());
+      TORCH_CHECK(norm_w->numel() == head_dim,
+                  "a per-head norm has one weight [head_dim]");
+    }
   } else if (norm_w.has_value()) {
     SEQ_F32(norm_w.value());
     TORCH_CHECK(norm_cols > 0 && norm_cols <= N &&
@@ -286,7 +343,7 @@ void norm_rope_rows(Tensor src, int64_t col, int64_t n_heads,
       head_norm ? 1 : 0, interleaved ? 1 : 0, (float)rot_mult,
       mix_src.has_value() ? mix_src->data_ptr() : nullptr, mix_ld,
       (int)mix_col, mix_lam.has_value() ? mix_lam->data_ptr() : nullptr,
-      seq_stream());
+      temp_coef, temp_every, seq_stream());
 }
 
 // checked options of the flexible attention beyond window / sink / cap
@@ -580,7 +637,10 @@ void register_seq_ops(pybind11::module& mod) {
   mod.def("rms_scale", &rms_scale, "x / rms(x) * g [* sigmoid(gate)]");
   mod.def("add_rms", &add_rms,
           "X += y on the fp32 residual; returns rms(X) * w (pre-norm)");
-  mod.def("gelu_gate", &gelu_gate, "gelu(gate) * up on a fused projection");
+  mod.def("act_gate", &act_gate,
+          "gelu / silu of the gate times up on a fused projection");
+  mod.def("head_rms_gate", &head_rms_gate,
+          "per-head RMS norm with a shared weight [* silu(gate)]");
   mod.def("gelu_mul", &gelu_mul,
           "GELU (erf or tanh form) times an optional gathered table slice");
   mod.def("soft_cap_", &soft_cap_, "cap * tanh(z / cap) in place");

@@ -9,7 +9,9 @@
 // the latent part of a latent row), rotate-half positions on a sub-range of
 // every head, then either a dense fp32 copy (queries) or a scatter into the
 // tokens' page rows (keys, values, latents). Angles are pos * f_i in double.
-// Options: the norm per head over the head's columns with one shared weight,
+// Options: the norm per head over the head's columns with one shared weight
+// (or none), a temperature 1 + coef ln(floor((pos + 1) / every) + 1) of the
+// token's position (queries of models without rotation),
 // rotation pairs (2i, 2i+1) instead of halves, a multiplier on cos and sin
 // (scaled rotations), and a blend (1 - lam) x + lam m with the same token's
 // columns of another projection (value mixing across layers) before the
@@ -64,14 +66,14 @@ __global__ __launch_bounds__(BLOCK) void norm_rope_rows_kernel(
     const int* __restrict__ table, int P, float* __restrict__ out,
     T* __restrict__ pool, int head_norm, int interleaved, float rot_mult,
     const T* __restrict__ mix_src, int mix_ld, int mix_col,
-    const float* __restrict__ mix_lam) {
+    const float* __restrict__ mix_lam, double temp_coef, double temp_every) {
   __shared__ float red[NWAVE];
   __shared__ float head_rn[MAX_NORM_HEADS];
   const int t = blockIdx.x;
   const int N = n_heads * head_dim;
   const T* row = src + (int64_t)t * ld + col;
   float rn = 1.f;
-  if (norm_w && head_norm) {
+  if (head_norm) {
     // one statistic per head, the weight [head_dim] shared by the heads
     const int lane = threadIdx.x & (WAVE_SIZE - 1);
     for (int hd = threadIdx.x / WAVE_SIZE; hd < n_heads; hd += NWAVE) {
@@ -95,6 +97,11 @@ __global__ __launch_bounds__(BLOCK) void norm_rope_rows_kernel(
   }
   const int pos = tok_pos[t];
   const int half = rot_dims / 2;
+  const float temp =
+      temp_every > 0.0
+          ? (float)(1.0 + temp_coef *
+                              log(floor((pos + 1) / temp_every) + 1.0))
+          : 1.f;
   int64_t prow = 0;
   if (pool) {
     const int page = table[(int64_t)tok_seq[t] * P + pos / PAGE];
@@ -104,10 +111,13 @@ __global__ __launch_bounds__(BLOCK) void norm_rope_rows_kernel(
   for (int c = threadIdx.x; c < N; c += BLOCK) {
     const int hd = c / head_dim, e = c - hd * head_dim;
     float x = ldv<T>(row + c);
-    if (norm_w) {
-      if (head_norm) x = x * head_rn[hd] * norm_w[e];
-      else if (c < norm_cols) x = x * rn * norm_w[c];
+    if (head_norm) {
+      x *= head_rn[hd];
+      if (norm_w) x *= norm_w[e];
+    } else if (norm_w && c < norm_cols) {
+      x = x * rn * norm_w[c];
     }
+    x *= temp;
     const int r = e - rot_off;
     if (r >= 0 && r < rot_dims) {
       // the pair's first member: r < half (halves) or r even (interleaved)
@@ -116,10 +126,13 @@ __global__ __launch_bounds__(BLOCK) void norm_rope_rows_kernel(
       const int step = interleaved ? 1 : half;
       const int cp = is_u ? c + step : c - step;       // the pair's other
       float y = ldv<T>(row + cp);
-      if (norm_w) {
-        if (head_norm) y = y * head_rn[hd] * norm_w[cp - hd * head_dim];
-        else if (cp < norm_cols) y = y * rn * norm_w[cp];
+      if (head_norm) {
+        y *= head_rn[hd];
+        if (norm_w) y *= norm_w[cp - hd * head_dim];
+      } else if (norm_w && cp < norm_cols) {
+        y = y * rn * norm_w[cp];
       }
+      y *= temp;
       const double ang = (double)pos * freqs[i];
       const float cs = (float)cos(ang) * rot_mult;
       const float sn = (float)sin(ang) * rot_mult;
@@ -469,6 +482,7 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        void* out, void* pool, int is_f32, int head_norm,
                        int interleaved, float rot_mult, const void* mix_src,
                        int mix_ld, int mix_col, const void* mix_lam,
+                       double temp_coef, double temp_every,
                        hipStream_t stream) {
   if (T <= 0) return;
   dim3 grid(T), block(BLOCK);
@@ -480,7 +494,7 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        (const int*)tok_pos, (const int*)table, P,
                        (float*)out, (float*)pool, head_norm, interleaved,
                        rot_mult, (const float*)mix_src, mix_ld, mix_col,
-                       (const float*)mix_lam);
+                       (const float*)mix_lam, temp_coef, temp_every);
   else
     hipLaunchKernelGGL(norm_rope_rows_kernel<bf16>, grid, block, 0, stream,
                        (const bf16*)src, ld, col, n_heads, head_dim,
@@ -489,7 +503,7 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        (const int*)tok_pos, (const int*)table, P,
                        (float*)out, (bf16*)pool, head_norm, interleaved,
                        rot_mult, (const bf16*)mix_src, mix_ld, mix_col,
-                       (const float*)mix_lam);
+                       (const float*)mix_lam, temp_coef, temp_every);
 }
 
 // heads per block for a shape: the largest of 8, 4, 2, 1 that divides the

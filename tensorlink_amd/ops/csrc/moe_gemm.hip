@@ -48,7 +48,8 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_gemm_kernel(
     const bf16* __restrict__ x,          // [T, K] (or [P, K] pair rows)
     const int* __restrict__ tok_idx,     // [P] row of x per pair, or null
     const int* __restrict__ seg_off,     // [E+1] pair segments by expert
-    const uint64_t* __restrict__ w_ptrs, // [E] -> weight [N, K]
+    const uint64_t* __restrict__ w_ptrs, // [E] -> weight [N, K], or null:
+    const bf16* __restrict__ w_base,     //   stacked [E, N, K] (bf16)
     const uint64_t* __restrict__ s_ptrs, // [E] -> fp32 scale [N] (FP8)
     bf16* __restrict__ out,              // [P, N]
     int N, int K) {
@@ -72,7 +73,9 @@ __global__ __launch_bounds__(BLOCK, 2) void moe_gemm_kernel(
   }
   __syncthreads();
 
-  const uint64_t wp = w_ptrs[e];
+  const uint64_t wp =
+      w_ptrs ? w_ptrs[e]
+             : reinterpret_cast<uint64_t>(w_base + (int64_t)e * N * K);
   const bf16* wrow_bf = FP8 ? nullptr
       : reinterpret_cast<const bf16*>(wp) + (int64_t)oc * K;
   const uint8_t* wrow_f8 = FP8
@@ -170,13 +173,23 @@ void tl_moe_gemm(const void* x, const void* tok_idx, const void* seg_off,
   if (fp8)
     hipLaunchKernelGGL((moe_gemm_kernel<1>), grid, block, 0, stream,
                        (const bf16*)x, (const int*)tok_idx,
-                       (const int*)seg_off, (const uint64_t*)w_ptrs,
+                       (const int*)seg_off, (const uint64_t*)w_ptrs, nullptr,
                        (const uint64_t*)s_ptrs, (bf16*)out, N, K);
   else
     hipLaunchKernelGGL((moe_gemm_kernel<0>), grid, block, 0, stream,
                        (const bf16*)x, (const int*)tok_idx,
                        (const int*)seg_off, (const uint64_t*)w_ptrs,
-                       nullptr, (bf16*)out, N, K);
+                       nullptr, nullptr, (bf16*)out, N, K);
+}
+
+// bf16 experts stacked in one tensor [E, N, K]
+void tl_moe_gemm_stacked(const void* x, const void* tok_idx,
+                         const void* seg_off, const void* w, void* out, int E,
+                         int N, int K, hipStream_t stream) {
+  dim3 grid(N / 64, E), block(BLOCK);
+  hipLaunchKernelGGL((moe_gemm_kernel<0>), grid, block, 0, stream,
+                     (const bf16*)x, (const int*)tok_idx, (const int*)seg_off,
+                     nullptr, (const bf16*)w, nullptr, (bf16*)out, N, K);
 }
 
 }  // extern "C"

@@ -13,8 +13,13 @@
 // Pre-norm layers use tl_add_rms: the previous sublayer's output is added
 // to the fp32 residual and the NEXT sublayer's input, rms(X) * w, is written
 // in the serving dtype by the same kernel (X <- X + y;  h = X / rms(X) * w).
-// tl_gelu_gate is the gated feed-forward's activation on a fused [gate | up]
-// projection: gelu(gate) * up.
+// A gated residual multiplies y element by element by the sigmoid of columns
+// of the sublayer's own projection in the same pass. Rows of a multiple of 4
+// columns are held in registers between the statistic and the scaling.
+// tl_act_gate is the gated feed-forward's activation on a fused [gate | up]
+// projection: act(gate) * up, act = gelu (erf / tanh form) or silu.
+// tl_head_rms_gate is the read-out norm of a linear-attention mixer whose
+// heads are normed on their own: x_h / rms(x_h) * w [* silu(gate)].
 
 #include "common.hpp"
 
@@ -62,19 +67,28 @@ __global__ __launch_bounds__(BLOCK) void postnorm_add_kernel(
   }
 }
 
+// y[c] [* sigmoid(gate[c])]
+template <typename T>
+DEVINLINE float gated(const T* y, const T* gate, int64_t c) {
+  const float v = ldf<T>(y, c);
+  return gate ? v / (1.f + expf(-ldf<T>(gate, c))) : v;
+}
+
 // X += y (if given); h = X / rms(X) * w in the serving dtype (no w: no h)
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void add_rms_kernel(
     float* __restrict__ X, const T* __restrict__ y,
     const float* __restrict__ w, T* __restrict__ h, int W, float eps,
-    float x_scale) {
+    float x_scale, const T* __restrict__ gate, int ldg) {
   __shared__ float red[NW];
   const int64_t row = blockIdx.x;
   float* xr = X + row * W;
+  const T* yr = y ? y + row * W : nullptr;
+  const T* gr = gate ? gate + row * ldg : nullptr;
   float ss = 0.f;
   for (int c = threadIdx.x; c < W; c += BLOCK) {
     float v = xr[c] * x_scale;
-    if (y) v += ldf<T>(y, row * W + c);
+    if (y) v += gated<T>(yr, gr, c);
     if (y || x_scale != 1.f) xr[c] = v;
     ss += v * v;
   }
@@ -86,34 +100,163 @@ __global__ __launch_bounds__(BLOCK) void add_rms_kernel(
     stf<T>(h, row * W + c, xr[c] * rn * w[c]);
 }
 
-// out[r][c] = gelu(p[r][c]) * p[r][N + c] on rows of 2N columns
+struct alignas(8) bf16x4 {
+  bf16 v[4];
+};
+DEVINLINE void ld4(const float* p, float (&o)[4]) {
+  const float4 x = *reinterpret_cast<const float4*>(p);
+  o[0] = x.x;
+  o[1] = x.y;
+  o[2] = x.z;
+  o[3] = x.w;
+}
+DEVINLINE void ld4(const bf16* p, float (&o)[4]) {
+  const bf16x4 x = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) o[e] = bf2f(x.v[e]);
+}
+DEVINLINE void st4(float* p, const float (&v)[4]) {
+  *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]);
+}
+DEVINLINE void st4(bf16* p, const float (&v)[4]) {
+  bf16x4 o;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) o.v[e] = f2bf(v[e]);
+  *reinterpret_cast<bf16x4*>(p) = o;
+}
+
+// the same for W a multiple of 4 and W <= 4 * BLOCK * NV: the row stays in
+// registers between the sum and the scaling
+template <typename T, int NV>
+__global__ __launch_bounds__(BLOCK) void add_rms_vec_kernel(
+    float* __restrict__ X, const T* __restrict__ y,
+    const float* __restrict__ w, T* __restrict__ h, int W, float eps,
+    float x_scale, const T* __restrict__ gate, int ldg) {
+  __shared__ float red[NW];
+  const int64_t row = blockIdx.x;
+  float* xr = X + row * W;
+  const T* yr = y ? y + row * W : nullptr;
+  const T* gr = gate ? gate + row * ldg : nullptr;
+  float v[NV][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = (k * BLOCK + threadIdx.x) * 4;
+    if (c < W) {
+      ld4(xr + c, v[k]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[k][e] *= x_scale;
+      if (y) {
+        float u[4];
+        ld4(yr + c, u);
+        if (gate) {
+          float g[4];
+          ld4(gr + c, g);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) u[e] = u[e] / (1.f + expf(-g[e]));
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[k][e] += u[e];
+      }
+      if (y || x_scale != 1.f) st4(xr + c, v[k]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += v[k][e] * v[k][e];
+    }
+  }
+  if (!w) return;
+  const float tot = block_reduce_sum<NW>(ss, red);
+  const float rn = 1.0f / sqrtf(tot / (float)W + eps);
+#pragma unroll
+  for (int k = 0; k < NV; ++k) {
+    const int c = (k * BLOCK + threadIdx.x) * 4;
+    if (c < W) {
+      float g[4];
+      ld4(w + c, g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[e] *= v[k][e] * rn;
+      st4(h + row * W + c, g);
+    }
+  }
+}
+
 template <typename T>
-__global__ __launch_bounds__(BLOCK) void gelu_gate_kernel(
-    const T* __restrict__ p, T* __restrict__ out, int64_t n, int N,
-    int tanh_form) {
+void launch_add_rms(float* X, const T* y, const float* w, T* h, int64_t rows,
+                    int W, float eps, float x_scale, const T* gate, int ldg,
+                    bool vec, hipStream_t stream) {
+  dim3 grid((unsigned)rows), block(BLOCK);
+#define TL_AR(NV)                                                           \
+  hipLaunchKernelGGL((add_rms_vec_kernel<T, NV>), grid, block, 0, stream, X, \
+                     y, w, h, W, eps, x_scale, gate, ldg)
+  const int nv = (W / 4 + BLOCK - 1) / BLOCK;
+  if (vec && nv <= 1) TL_AR(1);
+  else if (vec && nv <= 2) TL_AR(2);
+  else if (vec && nv <= 4) TL_AR(4);
+  else if (vec && nv <= 8) TL_AR(8);
+  else
+    hipLaunchKernelGGL(add_rms_kernel<T>, grid, block, 0, stream, X, y, w, h,
+                       W, eps, x_scale, gate, ldg);
+#undef TL_AR
+}
+
+// act(z): 0 erf GELU, 1 tanh-form GELU, 2 silu
+DEVINLINE float act_f(float z, int act) {
+  if (act == 2) return z / (1.f + expf(-z));
+  return gelu_f(z, act);
+}
+
+// out[r][c] = act(p[r][c]) * p[r][N + c] on rows of stride ld
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void act_gate_kernel(
+    const T* __restrict__ p, int64_t ld, T* __restrict__ out, int64_t n,
+    int N, int act) {
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n;
        i += (int64_t)gridDim.x * BLOCK) {
     const int64_t r = i / N;
     const int c = (int)(i - r * N);
-    const T* row = p + r * 2 * N;
-    stf<T>(out, i, gelu_f(ldf<T>(row, c), tanh_form) * ldf<T>(row, N + c));
+    const T* row = p + r * ld;
+    stf<T>(out, i, act_f(ldf<T>(row, c), act) * ldf<T>(row, N + c));
   }
 }
 
-// bf16 rows whose half width is a multiple of 8: 16-byte loads and stores
-__global__ __launch_bounds__(BLOCK) void gelu_gate_vec8_kernel(
-    const bf16x8* __restrict__ p, bf16x8* __restrict__ out, int64_t n8,
-    int N8, int tanh_form) {
+// bf16, N, the stride and the first column multiples of 8: 16-byte accesses
+__global__ __launch_bounds__(BLOCK) void act_gate_vec8_kernel(
+    const bf16x8* __restrict__ p, int64_t ld8, bf16x8* __restrict__ out,
+    int64_t n8, int N8, int act) {
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n8;
        i += (int64_t)gridDim.x * BLOCK) {
     const int64_t r = i / N8;
     const int c = (int)(i - r * N8);
-    const bf16x8 a = p[r * 2 * N8 + c], b = p[r * 2 * N8 + N8 + c];
+    const bf16x8 a = p[r * ld8 + c], b = p[r * ld8 + N8 + c];
     bf16x8 o;
 #pragma unroll
     for (int e = 0; e < 8; ++e)
-      o.v[e] = f2bf(gelu_f(bf2f(a.v[e]), tanh_form) * bf2f(b.v[e]));
+      o.v[e] = f2bf(act_f(bf2f(a.v[e]), act) * bf2f(b.v[e]));
     out[i] = o;
+  }
+}
+
+// one wave per (row, head): out = x_h / rms(x_h) * w [* silu(gate)]
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void head_rms_gate_kernel(
+    const float* __restrict__ x, const float* __restrict__ w,
+    const T* __restrict__ gate, int ldg, T* __restrict__ out, int64_t units,
+    int H, int V, float eps) {
+  const int64_t u = (int64_t)blockIdx.x * NW + threadIdx.x / WAVE_SIZE;
+  if (u >= units) return;
+  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+  const float* xr = x + u * V;
+  float ss = 0.f;
+  for (int c = lane; c < V; c += WAVE_SIZE) ss += xr[c] * xr[c];
+  ss = wave_reduce_sum(ss);
+  const float rn = 1.0f / sqrtf(ss / (float)V + eps);
+  const T* gr = gate ? gate + (u / H) * ldg + (u % H) * V : nullptr;
+  for (int c = lane; c < V; c += WAVE_SIZE) {
+    float v = xr[c] * rn * w[c];
+    if (gate) {
+      const float z = ldf<T>(gr, c);
+      v *= z / (1.f + expf(-z));
+    }
+    stf<T>(out, u * V + c, v);
   }
 }
 
@@ -171,11 +314,15 @@ __global__ __launch_bounds__(BLOCK) void gelu_vec8_kernel(
   }
 }
 
+// cap 0: the scale alone
 __global__ __launch_bounds__(BLOCK) void soft_cap_kernel(float* z, int64_t n,
-                                                         float cap) {
+                                                         float cap,
+                                                         float scale) {
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n;
-       i += (int64_t)gridDim.x * BLOCK)
-    z[i] = cap * tanhf(z[i] / cap);
+       i += (int64_t)gridDim.x * BLOCK) {
+    const float v = z[i] * scale;
+    z[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
+  }
 }
 
 int ew_grid(int64_t n) {
@@ -202,38 +349,57 @@ void tl_postnorm_add(void* X, const void* y, const void* w, void* h,
                        W, eps, one_plus);
 }
 
+// gate: first gate column of row 0 (rows of stride ldg), or null
 void tl_add_rms(void* X, const void* y, const void* w, void* h, int64_t rows,
-                int W, float eps, float x_scale, int is_f32,
-                hipStream_t stream) {
+                int W, float eps, float x_scale, const void* gate, int ldg,
+                int gate_aligned, int is_f32, hipStream_t stream) {
   if (rows <= 0) return;
-  dim3 grid((unsigned)rows), block(BLOCK);
+  const bool vec = W % 4 == 0 && (!gate || gate_aligned);
   if (is_f32)
-    hipLaunchKernelGGL(add_rms_kernel<float>, grid, block, 0, stream,
-                       (float*)X, (const float*)y, (const float*)w, (float*)h,
-                       W, eps, x_scale);
+    launch_add_rms<float>((float*)X, (const float*)y, (const float*)w,
+                          (float*)h, rows, W, eps, x_scale,
+                          (const float*)gate, ldg, vec, stream);
   else
-    hipLaunchKernelGGL(add_rms_kernel<bf16>, grid, block, 0, stream,
-                       (float*)X, (const bf16*)y, (const float*)w, (bf16*)h,
-                       W, eps, x_scale);
+    launch_add_rms<bf16>((float*)X, (const bf16*)y, (const float*)w, (bf16*)h,
+                         rows, W, eps, x_scale, (const bf16*)gate, ldg, vec,
+                         stream);
 }
 
-void tl_gelu_gate(const void* p, void* out, int64_t rows, int N,
-                  int tanh_form, int is_f32, hipStream_t stream) {
+// p: first gate column of row 0, rows of stride ld
+void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
+                 int64_t rows, int N, int act, int is_f32,
+                 hipStream_t stream) {
   const int64_t n = rows * N;
   if (n <= 0) return;
-  if (!is_f32 && N % 8 == 0) {
-    hipLaunchKernelGGL(gelu_gate_vec8_kernel, dim3(ew_grid(n / 8)),
-                       dim3(BLOCK), 0, stream, (const bf16x8*)p, (bf16x8*)out,
-                       n / 8, N / 8, tanh_form);
+  if (!is_f32 && aligned && N % 8 == 0) {
+    hipLaunchKernelGGL(act_gate_vec8_kernel, dim3(ew_grid(n / 8)),
+                       dim3(BLOCK), 0, stream, (const bf16x8*)p, ld / 8,
+                       (bf16x8*)out, n / 8, N / 8, act);
     return;
   }
   dim3 grid(ew_grid(n)), block(BLOCK);
   if (is_f32)
-    hipLaunchKernelGGL(gelu_gate_kernel<float>, grid, block, 0, stream,
-                       (const float*)p, (float*)out, n, N, tanh_form);
+    hipLaunchKernelGGL(act_gate_kernel<float>, grid, block, 0, stream,
+                       (const float*)p, ld, (float*)out, n, N, act);
   else
-    hipLaunchKernelGGL(gelu_gate_kernel<bf16>, grid, block, 0, stream,
-                       (const bf16*)p, (bf16*)out, n, N, tanh_form);
+    hipLaunchKernelGGL(act_gate_kernel<bf16>, grid, block, 0, stream,
+                       (const bf16*)p, ld, (bf16*)out, n, N, act);
+}
+
+void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
+                      void* out, int64_t rows, int H, int V, float eps,
+                      int is_f32, hipStream_t stream) {
+  const int64_t units = rows * H;
+  if (units <= 0) return;
+  dim3 grid((unsigned)((units + NW - 1) / NW)), block(BLOCK);
+  if (is_f32)
+    hipLaunchKernelGGL(head_rms_gate_kernel<float>, grid, block, 0, stream,
+                       (const float*)x, (const float*)w, (const float*)gate,
+                       ldg, (float*)out, units, H, V, eps);
+  else
+    hipLaunchKernelGGL(head_rms_gate_kernel<bf16>, grid, block, 0, stream,
+                       (const float*)x, (const float*)w, (const bf16*)gate,
+                       ldg, (bf16*)out, units, H, V, eps);
 }
 
 void tl_rms_scale(const void* x, const void* w, const void* gate, int ldg,
@@ -274,10 +440,11 @@ void tl_gelu(const void* x, void* out, int64_t n, int N, int tanh_form,
                        (const int*)tokens);
 }
 
-void tl_soft_cap(void* z, int64_t n, float cap, hipStream_t stream) {
+void tl_soft_cap(void* z, int64_t n, float cap, float scale,
+                 hipStream_t stream) {
   if (n <= 0) return;
   hipLaunchKernelGGL(soft_cap_kernel, dim3(ew_grid(n)), dim3(BLOCK), 0,
-                     stream, (float*)z, n, cap);
+                     stream, (float*)z, n, cap, scale);
 }
 
 }  // extern "C"

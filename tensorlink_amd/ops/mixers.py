@@ -390,10 +390,24 @@ def postnorm_add(X: torch.Tensor, y: torch.Tensor, w: torch.Tensor,
 
 def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float, one_plus: bool,
               gate: Optional[torch.Tensor] = None, gate_col: int = 0,
-              out_dtype=torch.float32) -> torch.Tensor:
+              out_dtype=torch.float32, heads: int = 0) -> torch.Tensor:
     """x / rms(x) * (1 + w | w) over the last axis of x [T, N] (fp32),
-    optionally times sigmoid(gate[:, gate_col:gate_col + N])."""
+    optionally times sigmoid(gate[:, gate_col:gate_col + N]). With ``heads``
+    > 0 every one of that many equal parts of a row has its own statistic,
+    the weight [N / heads] is shared by them, and the gate goes through
+    silu instead of the sigmoid."""
     assert x.dtype == torch.float32 and w.dtype == torch.float32
+    if heads:
+        assert not one_plus and x.shape[1] == heads * w.numel()
+        if x.is_cuda:
+            return _ext().head_rms_gate(
+                x.contiguous(), w, int(heads), float(eps), gate,
+                int(gate_col), out_dtype == torch.float32)
+        y = (_rms(x.view(x.shape[0], heads, -1), eps) * w).reshape(x.shape)
+        if gate is not None:
+            y = y * torch.nn.functional.silu(
+                gate[:, gate_col:gate_col + x.shape[1]].float())
+        return y.to(out_dtype)
     if x.is_cuda:
         return _ext().rms_scale(x.contiguous(), w, float(eps),
                                 bool(one_plus), gate, int(gate_col),
@@ -423,46 +437,94 @@ def gelu(x: torch.Tensor, tanh_form: bool = False,
     return y.to(x.dtype)
 
 
-def soft_cap_(z: torch.Tensor, cap: float) -> torch.Tensor:
-    """cap * tanh(z / cap) in place on fp32 logits."""
+def soft_cap_(z: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
+    """cap * tanh(z * scale / cap) in place on fp32 logits; cap 0 = no cap
+    (only the scale)."""
     assert z.dtype == torch.float32
     if z.is_cuda:
-        _ext().soft_cap_(z, float(cap))
+        _ext().soft_cap_(z, float(cap), float(scale))
         return z
-    return z.copy_(cap * torch.tanh(z / cap))
+    z *= scale
+    return z.copy_(cap * torch.tanh(z / cap)) if cap else z
 
 
 def add_rms(X: torch.Tensor, y: Optional[torch.Tensor],
             w: Optional[torch.Tensor], eps: float, out_dtype=torch.float32,
-            x_scale: float = 1.0) -> torch.Tensor:
+            x_scale: float = 1.0, gate: Optional[torch.Tensor] = None,
+            gate_col: int = 0) -> torch.Tensor:
     """Pre-norm residual step, in place on the fp32 residual X [T, W]:
     X <- X * x_scale + y (``y`` = the previous sublayer's output, or None),
     then returns the next sublayer's input X / rms(X) * w in ``out_dtype``;
     without ``w`` (after the last sublayer) only the add is done and X is
-    returned. Sum, statistic and scaling are fp32."""
+    returned. With ``gate`` [T, L] y is first multiplied, element by
+    element, by sigmoid(gate[:, gate_col:gate_col + W]) (a gated residual;
+    the pre-activations are columns of the sublayer's own projection).
+    Sum, sigmoid, statistic and scaling are fp32."""
     assert X.dtype == torch.float32
     assert w is None or w.dtype == torch.float32
+    assert gate is None or y is not None
     if X.is_cuda:
         return _ext().add_rms(
             X, None if y is None else y.contiguous(), w, float(eps),
-            float(x_scale), out_dtype == torch.float32)
+            float(x_scale), gate, int(gate_col),
+            out_dtype == torch.float32)
     if x_scale != 1.0:
         X *= x_scale
     if y is not None:
-        X += y.float()
+        u = y.float()
+        if gate is not None:
+            u = u * torch.sigmoid(
+                gate[:, gate_col:gate_col + X.shape[1]].float())
+        X += u
     return X if w is None else (_rms(X, eps) * w).to(out_dtype)
+
+
+GATE_ACTS = {"gelu": 0, "gelu_tanh": 1, "silu": 2}
+
+
+def act_gate(p: torch.Tensor, act: str, N: int = 0,
+             col: int = 0) -> torch.Tensor:
+    """act(p[:, col:col + N]) * p[:, col + N:col + 2N] for a fused
+    projection p [T, L] that holds [gate | up] from column ``col`` (N = 0:
+    the whole of p); ``act`` is "gelu" (erf), "gelu_tanh" or "silu".
+    Evaluated in fp32, result [T, N] in p's dtype."""
+    N = N or p.shape[1] // 2
+    if p.is_cuda:
+        return _ext().act_gate(p.contiguous(), int(col), int(N),
+                               GATE_ACTS[act])
+    g = p[:, col:col + N].float()
+    F = torch.nn.functional
+    y = F.silu(g) if act == "silu" else F.gelu(
+        g, approximate="tanh" if act == "gelu_tanh" else "none")
+    return (y * p[:, col + N:col + 2 * N].float()).to(p.dtype)
 
 
 def gelu_gate(p: torch.Tensor, tanh_form: bool = True) -> torch.Tensor:
     """gelu(p[:, :N]) * p[:, N:] for a fused [gate | up] projection
     p [T, 2N]; evaluated in fp32, result in p's dtype."""
-    if p.is_cuda:
-        return _ext().gelu_gate(p.contiguous(), bool(tanh_form))
-    N = p.shape[1] // 2
-    f = p.float()
-    y = torch.nn.functional.gelu(
-        f[:, :N], approximate="tanh" if tanh_form else "none") * f[:, N:]
-    return y.to(p.dtype)
+    return act_gate(p, "gelu_tanh" if tanh_form else "gelu")
+
+
+def pair_linear(X: torch.Tensor, Y: torch.Tensor, W: torch.Tensor,
+                base: Optional[torch.Tensor] = None):
+    """W [x; y] for W [N, A + B] applied to fp32 rows X [T, A] beside rows
+    Y [T, B], as two products with fp32 results: the operands are rounded
+    to W's dtype, the sums are not. ``base`` is the y part of an earlier
+    call with the same Y and W; returns (W [x; y], y part)."""
+    A = X.shape[1]
+    wx, wy = W[:, :A].t(), W[:, A:].t()
+
+    def prod(a, b):
+        a = a.to(W.dtype)
+        if W.dtype == torch.float32:
+            return a @ b
+        if a.is_cuda:
+            return torch.mm(a, b, out_dtype=torch.float32)
+        return a.float() @ b.float()
+
+    if base is None:
+        base = prod(Y, wy)
+    return prod(X, wx) + base, base
 
 
 # ---------------------------------------------------------------------------
@@ -485,11 +547,14 @@ def norm_rope_rows(src: torch.Tensor, col: int, n_heads: int, head_dim: int,
                    head_norm: bool = False, interleaved: bool = False,
                    rot_mult: float = 1.0,
                    mix_src: Optional[torch.Tensor] = None, mix_col: int = 0,
-                   mix_lam: Optional[torch.Tensor] = None):
+                   mix_lam: Optional[torch.Tensor] = None,
+                   temp: Optional[Sequence[float]] = None):
     """Take columns [col, col + n_heads*head_dim) of src [T, L]; RMS-norm
     the first ``norm_cols`` of them together (weight ``norm_w``, plain) or,
     with ``head_norm``, every head on its own with the one weight
-    [head_dim]; rotate dims [rot_off, rot_off + rot_dims) of every head by
+    [head_dim] (no ``norm_w``: a weight of one); multiply by the position
+    temperature 1 + coef ln(floor((pos + 1) / every) + 1) for ``temp`` =
+    (coef, every); rotate dims [rot_off, rot_off + rot_dims) of every head by
     the token's position (pairs (i, i + rot_dims/2), or (2i, 2i+1) with
     ``interleaved``; angle pos * freqs[i]; cos and sin times ``rot_mult``);
     with ``mix_src`` blend the result with the same token's columns
@@ -509,17 +574,21 @@ def norm_rope_rows(src: torch.Tensor, col: int, n_heads: int, head_dim: int,
                               meta.tok_seq, meta.tok_pos, meta.table, out,
                               pool, bool(head_norm), bool(interleaved),
                               float(rot_mult), mix_src, int(mix_col),
-                              mix_lam)
+                              mix_lam, float(temp[0]) if temp else 0.0,
+                              float(temp[1]) if temp else 0.0)
         return out
     x = src[:, col:col + N].float()
-    if norm_w is not None and head_norm:
-        x = (_rms(x.reshape(T, n_heads, head_dim), eps)
-             * norm_w).reshape(T, N)
+    if head_norm:
+        x = _rms(x.reshape(T, n_heads, head_dim), eps)
+        x = (x if norm_w is None else x * norm_w).reshape(T, N)
     elif norm_w is not None:
         x = torch.cat([_rms(x[:, :norm_cols], eps) * norm_w,
                        x[:, norm_cols:]], 1)
     x = x.reshape(T, n_heads, head_dim).clone()
     pos = meta.tok_pos.long()
+    if temp:
+        n = torch.floor((pos.double() + 1.0) / float(temp[1])) + 1.0
+        x *= (1.0 + float(temp[0]) * torch.log(n)).float().view(T, 1, 1)
     if rot_dims:
         half = rot_dims // 2
         ang = pos.double().view(T, 1, 1) * freqs.double().view(1, 1, half)
@@ -1034,3 +1103,123 @@ def polynorm(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
     out = (coef[0] * _rms(f, eps) + coef[1] * _rms(f2, eps)
            + coef[2] * _rms(f2 * f, eps) + coef[3])
     return out.to(z.dtype)
+
+
+# ---------------------------------------------------------------------------
+# gated linear attention: outer-product memory with one decay per key
+# channel and token
+# ---------------------------------------------------------------------------
+def gla_chunk(D: int) -> int:
+    """Tokens per chunk of the chunk form of the gated linear attention for
+    key size D; 0 if the chunk kernels do not serve it."""
+    return 64 if D <= 128 else 32 if D <= 256 else 0
+
+
+def gla_scan(proj: torch.Tensor, offs, a2t: torch.Tensor, bias: torch.Tensor,
+             tau: float, S: torch.Tensor, meta: RaggedMeta, H: int, D: int,
+             V: int) -> torch.Tensor:
+    """Per head: S_t = diag(alpha_t) S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.
+
+    proj [T, L] holds q [H*D] | k [H*D] | v [H*V] | r [R] at columns
+    ``offs``; q is scaled by D^-1/2. alpha = sigmoid(z)^(1/tau) with
+    z = r a2t + bias (a2t [R, H*D], bias [H*D], fp32). The state pool
+    S [slots, H, D, V] (fp32) is read at ``meta.slots`` (zeros for a sequence
+    with no cached tokens) and written back. Everything after the
+    projection is fp32; returns the raw read-out [T, H*V] in fp32."""
+    q_off, k_off, v_off, r_off = (int(x) for x in offs)
+    T, R = proj.shape[0], a2t.shape[0]
+    assert a2t.dtype == bias.dtype == S.dtype == torch.float32
+    assert a2t.shape[1] == bias.numel() == H * D
+    if proj.is_cuda:
+        C = gla_chunk(D)
+        if (C and max(meta.new_h) >= 2 * C
+                and not os.environ.get("TL_NO_SCAN_CHUNKS")
+                and T * H * D * V * 4 // C <= (1 << 33)
+                and _ext().gla_chunks_ok(int(D), int(R), C)):
+            # long prompt portions: chunk summaries, the chain over them,
+            # then every chunk's read-out (all chunks in parallel)
+            cu_c, _, _, base, cnt, nc, _ = meta.scan_chunks(C)
+            return _ext().gla_chunks(proj, q_off, k_off, v_off, r_off, a2t,
+                                     bias, float(tau), S, cu_c, base, cnt,
+                                     meta.slots, meta.pos0, int(H), int(D),
+                                     int(V), int(C))
+        return _ext().gla_scan(proj, q_off, k_off, v_off, r_off, a2t, bias,
+                               float(tau), S, meta.cu, meta.slots, meta.pos0,
+                               int(H), int(D), int(V))
+    pf = proj.float()
+    q = pf[:, q_off:q_off + H * D].view(T, H, D) * D ** -0.5
+    k = pf[:, k_off:k_off + H * D].view(T, H, D)
+    v = pf[:, v_off:v_off + H * V].view(T, H, V)
+    z = pf[:, r_off:r_off + R] @ a2t + bias
+    alpha = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(T, H, D)
+    o = torch.empty(T, H, V)
+    for b in range(meta.B):
+        t0, t1 = meta.cu_h[b], meta.cu_h[b + 1]
+        if t1 == t0:
+            continue
+        slot = meta.slots_h[b]
+        Sb = (torch.zeros(H, D, V) if meta.pos0_h[b] == 0
+              else S[slot].clone())
+        for t in range(t0, t1):
+            Sb = alpha[t].unsqueeze(-1) * Sb + k[t].unsqueeze(-1) \
+                * v[t].unsqueeze(1)
+            o[t] = (Sb * q[t].unsqueeze(-1)).sum(1)
+        S[slot] = Sb
+    return o.reshape(T, H * V)
+
+
+# ---------------------------------------------------------------------------
+# mixture of experts without groups: fp32 router, softmax over the chosen
+# logits, expert-sorted grouped products, weighted combine
+# ---------------------------------------------------------------------------
+def topk_softmax_router(h: torch.Tensor, w: torch.Tensor, top: int):
+    """Logits z = w h in fp32 (w [E, W] fp32); the ``top`` largest are
+    chosen (the lower index wins a tie) and weighted by the softmax over
+    the chosen logits only. Returns (weights [T, top] fp32, indices
+    [T, top] int32)."""
+    assert w.dtype == torch.float32
+    if h.is_cuda:
+        # few rows: the logits are computed by the selecting kernel itself
+        z = (torch.nn.functional.linear(h.float(), w)
+             if h.shape[0] > 64 else None)
+        wt, idx = _ext().moe_route(h.contiguous(), w, z, int(top))
+        return wt, idx
+    z = torch.nn.functional.linear(h.float(), w)
+    idx = torch.sort(z, dim=-1, descending=True, stable=True).indices[:, :top]
+    return torch.softmax(z.gather(1, idx), -1), idx.to(torch.int32)
+
+
+def expert_gated_ff(h: torch.Tensor, wts: torch.Tensor, idx: torch.Tensor,
+                    gate_up: torch.Tensor, down: torch.Tensor, act: str, *,
+                    shared: Optional[torch.Tensor] = None,
+                    sgate: Optional[torch.Tensor] = None,
+                    sgate_col: int = 0) -> torch.Tensor:
+    """sum_j wts[:, j] E_idx[:, j](h), E_e(x) = down_e(act(gate_e x) *
+    (up_e x)), plus ``shared`` [T, W] times sigmoid(sgate[:, sgate_col]).
+    gate_up [E, 2 ff, W] and down [E, W, ff] are the stacked experts; their
+    products run in h's dtype with fp32 accumulation, the weighted sum is
+    fp32; result in h's dtype."""
+    T, W = h.shape
+    E, ff = gate_up.shape[0], gate_up.shape[1] // 2
+    top = idx.shape[1]
+    if h.is_cuda:
+        C = _ext()
+        seg, pair_tok, rank = C.moe_sort(idx, E)
+        a = C.moe_gemm_stacked(h.contiguous(), pair_tok, seg, gate_up)
+        y = C.moe_gemm_stacked(act_gate(a, act), None, seg, down)
+        return C.moe_combine(y, rank, wts, shared, sgate, int(sgate_col))
+    out = torch.zeros(T, W, dtype=torch.float32)
+    for e in range(E):
+        tok, choice = (idx == e).nonzero(as_tuple=True)
+        if tok.numel() == 0:
+            continue
+        a = act_gate(torch.nn.functional.linear(h[tok], gate_up[e]), act)
+        out.index_add_(0, tok, torch.nn.functional.linear(
+            a, down[e]).float() * wts[tok, choice, None])
+    if shared is not None:
+        s = shared.float()
+        if sgate is not None:
+            s = s * torch.sigmoid(
+                sgate[:, sgate_col:sgate_col + 1].float())
+        out += s
+    return out.to(h.dtype)
