@@ -50,11 +50,13 @@ def parse_args():
     p.add_argument("--sizes", default="w1024,w2048",
                    help="layered mode: comma list of size presets")
     p.add_argument("--family",
-                   choices=["kepusun", "senulix", "dizepel", "potosun"],
+                   choices=["kepusun", "senulix", "dizepel", "potosun",
+                            "mogisun"],
                    default="kepusun",
                    help="layered mode: which layered family to time "
                         "(senulix, dizepel: beside an equal-size dense GQA "
                         "decoder; potosun: beside an equal-size Senulix "
+                        "model; mogisun: beside an equal-size Kepusun "
                         "model)")
     p.add_argument("--dp", type=int, default=1,
                    help="data-parallel replicas (train mode; world=dp*pp)")
@@ -307,6 +309,59 @@ def potosun_configs(z):
     return pot, sen
 
 
+MOGISUN_SIZES = {
+    # layers: attention, gla, attention, gla; the middle two run twice
+    "w1024": dict(width=1024, heads=8, kv=2, dim=64, vdim=128, rank=16,
+                  experts=16, top=2, ff=320, kep_ff=512, vocab=32000,
+                  batch=8, prompt=2048),
+    "w2048": dict(width=2048, heads=16, kv=4, dim=64, vdim=128, rank=16,
+                  experts=32, top=4, ff=512, kep_ff=768, vocab=32000,
+                  batch=8, prompt=2048),
+    "tiny": dict(width=128, heads=2, kv=1, dim=32, vdim=64, rank=8,
+                 experts=4, top=2, ff=64, kep_ff=96, vocab=512, batch=2,
+                 prompt=96),
+}
+
+
+def mogisun_configs(z):
+    """(Mogisun config, Kepusun config) of a preset: same width, vocabulary,
+    heads, recurrent state per head, attention key and value width, expert
+    count and top; Kepusun has as many layers as Mogisun has layer RUNS, and
+    Mogisun's gated three-matrix experts get about 2/3 of the width of
+    Kepusun's two-matrix ones (Mogisun has a shared expert besides)."""
+    from tensorlink_amd.models.kepusun import KepusunConfig
+    from tensorlink_amd.models.mogisun import MogisunConfig
+    H, D, V, kv = z["heads"], z["dim"], z["vdim"], z["kv"]
+    router = {"experts": z["experts"], "top": z["top"]}
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"]}, "router": router,
+           "shared": {"ff": z["ff"]}}
+    at = {"type": "attention", "mlp": mlp, "mixer": {
+        "heads": H, "kv_heads": kv, "dim": 2 * D, "vdim": V,
+        "scale": (2 * D) ** -0.5, "q_temp": {"coef": 0.2, "every": 1024}}}
+    gl = {"type": "gla", "mlp": mlp, "mixer": {
+        "heads": H, "dim": D, "vdim": V, "tau": 12.0,
+        "decay_rank": z["rank"]}}
+    mog = MogisunConfig.from_dict({
+        "architecture": "Mogisun", "vocab": z["vocab"], "width": z["width"],
+        "norm": {"eps": 1e-6}, "logit_scale": 0.5, "logit_softcap": 30.0,
+        "loop": {"start": 1, "stop": 3, "times": 2},
+        "layers": [at, gl, at, gl]}, name="mogisun-" + str(z["width"]))
+    kmlp = {"kind": "moe", "expert": {"ff": z["kep_ff"]},
+            "router": dict(router, scale=1.0,
+                           groups={"count": 4, "keep": 2})}
+    km = {"type": "mlstm", "mlp": kmlp,
+          "mixer": {"heads": H, "dim": D, "vdim": V, "gate_cap": 15.0}}
+    ka = {"type": "attention", "mlp": kmlp, "mixer": {
+        "heads": H, "kv_heads": kv, "dim": D, "vdim": V,
+        "scale": D ** -0.5, "diff": 0.5}}
+    kep = KepusunConfig.from_dict({
+        "architecture": "Kepusun", "vocab": z["vocab"],
+        "width": z["width"], "streams": 2, "norm": {"eps": 1e-6},
+        "layers": [ka, km, ka, km, ka, km]},
+        name="kepusun-" + str(z["width"]))
+    return mog, kep
+
+
 @torch.no_grad()
 def run_layered(args, device, use_gpu):
     """Prefill and decode tokens/s of the Kepusun family beside the
@@ -356,7 +411,17 @@ def run_layered(args, device, use_gpu):
         return out
 
     for name in args.sizes.split(","):
-        if args.family == "potosun":
+        if args.family == "mogisun":
+            z = MOGISUN_SIZES[name]
+            mog, kep = mogisun_configs(z)
+            B, S = z["batch"], z["prompt"]
+            only = os.environ.get("TL_BENCH_ONLY")     # profile one model
+            res = {}
+            if only in (None, "mogisun"):
+                res["mogisun"] = measure(mog, B, S)
+            if only in (None, "kepusun"):
+                res["kepusun"] = measure(kep, B, S)
+        elif args.family == "potosun":
             z = POTOSUN_SIZES[name]
             pot, sen = potosun_configs(z)
             B, S = z["batch"], z["prompt"]
