@@ -35,6 +35,15 @@ void tl_grouped_any(const void* x, const void* tok_idx, const void* seg,
 void tl_moe_gemm_stacked(const void* x, const void* tok_idx,
                          const void* seg_off, const void* w, void* out, int E,
                          int N, int K, hipStream_t stream);
+void tl_moe_tiles(const void* x, const void* tok, const void* seg,
+                  const void* w, void* out, int P, int E, int N, int K,
+                  hipStream_t stream);
+void tl_moe_rows(const void* x, const void* tok, const void* seg,
+                 const void* w, void* out, int P, int E, int N, int K,
+                 hipStream_t stream);
+void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
+                 int64_t rows, int N, int act, int is_f32,
+                 hipStream_t stream);
 void tl_moe_combine(const void* y, const void* rank, const void* wt,
                     const void* shared, const void* sg, int ldg, int sg_col,
                     void* out, int64_t T, int W, int top, int is_f32,
@@ -218,7 +227,15 @@ Tensor moe_gemm_stacked(Tensor x, c10::optional<Tensor> tok, Tensor seg,
   const int64_t E = w.size(0), N = w.size(1), K = w.size(2);
   auto out = torch::empty({P, N}, x.options());
   if (P == 0) return out;
-  if (!is_f32 && K % 32 == 0 && N % 64 == 0)
+  const bool mfma = !is_f32 && K % 32 == 0 && N % 64 == 0;
+  if (mfma && P <= 128)
+    tl_moe_rows(x.data_ptr(), ti, seg.data_ptr(), w.data_ptr(),
+                out.data_ptr(), (int)P, (int)E, (int)N, (int)K, gla_stream());
+  else if (mfma && P >= 64 * E && P >= 1024)
+    tl_moe_tiles(x.data_ptr(), ti, seg.data_ptr(), w.data_ptr(),
+                 out.data_ptr(), (int)P, (int)E, (int)N, (int)K,
+                 gla_stream());
+  else if (mfma)
     tl_moe_gemm_stacked(x.data_ptr(), ti, seg.data_ptr(), w.data_ptr(),
                         out.data_ptr(), (int)E, (int)N, (int)K, gla_stream());
   else
@@ -265,6 +282,27 @@ Tensor moe_combine(Tensor y, Tensor rank, Tensor wt,
   return out;
 }
 
+// the routed experts of a step in one call: sort, gate|up product,
+// activation, down product, combine (gate_up [E, 2 ff, W], down [E, W, ff])
+Tensor moe_experts(Tensor h, Tensor wt, Tensor idx, Tensor gate_up,
+                   Tensor down, int64_t act, c10::optional<Tensor> shared,
+                   c10::optional<Tensor> sg, int64_t sg_col) {
+  TORCH_CHECK(gate_up.dim() == 3 && down.dim() == 3 && h.dim() == 2 &&
+                  gate_up.size(1) == 2 * down.size(2) &&
+                  gate_up.size(0) == down.size(0) &&
+                  down.size(1) == h.size(1) && idx.dim() == 2 &&
+                  idx.size(0) == h.size(0) && act >= 0 && act <= 2,
+              "h [T, W], idx [T, top], gate_up [E, 2 ff, W], down [E, W, ff]");
+  auto s = moe_sort(idx, gate_up.size(0));
+  Tensor a = moe_gemm_stacked(h, s[1], s[0], gate_up);
+  const int64_t ff = down.size(2);
+  auto b = torch::empty({a.size(0), ff}, a.options());
+  tl_act_gate(a.data_ptr(), 2 * ff, ff % 8 == 0, b.data_ptr(), a.size(0),
+              (int)ff, (int)act, gla_is_f32(a), gla_stream());
+  Tensor y = moe_gemm_stacked(b, c10::nullopt, s[0], down);
+  return moe_combine(y, s[2], wt, shared, sg, sg_col);
+}
+
 }  // namespace
 
 void register_gla_ops(pybind11::module& mod) {
@@ -279,6 +317,8 @@ void register_gla_ops(pybind11::module& mod) {
   mod.def("moe_sort", &moe_sort, "expert-sorted (token, choice) pairs");
   mod.def("moe_gemm_stacked", &moe_gemm_stacked,
           "grouped product with stacked experts, any size, bf16 or fp32");
+  mod.def("moe_experts", &moe_experts,
+          "sort, grouped products, activation and combine in one call");
   mod.def("moe_combine", &moe_combine,
           "weighted sum of a token's experts plus a gated shared expert");
 }

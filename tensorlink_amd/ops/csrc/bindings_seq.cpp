@@ -25,8 +25,8 @@ void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
                  int64_t rows, int N, int act, int is_f32,
                  hipStream_t stream);
 void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
-                      void* out, int64_t rows, int H, int V, float eps,
-                      int is_f32, hipStream_t stream);
+                      int gate_aligned, void* out, int64_t rows, int H, int V,
+                      float eps, int is_f32, hipStream_t stream);
 void tl_gelu(const void* x, void* out, int64_t n, int N, int tanh_form,
              const void* table, int ldt, int table_col, const void* tokens,
              int is_f32, hipStream_t stream);
@@ -224,7 +224,8 @@ Tensor head_rms_gate(Tensor x, Tensor w, int64_t H, double eps,
   auto out = torch::empty(
       x.sizes(),
       x.options().dtype(out_f32 ? torch::kFloat : torch::kBFloat16));
-  tl_head_rms_gate(x.data_ptr(), w.data_ptr(), gp, ldg, out.data_ptr(),
+  tl_head_rms_gate(x.data_ptr(), w.data_ptr(), gp, ldg,
+                   ldg % 4 == 0 && gate_col % 4 == 0, out.data_ptr(),
                    x.size(0), (int)H, (int)V, (float)eps, out_f32 ? 1 : 0,
                    seq_stream());
   return out;

@@ -422,21 +422,25 @@ __global__ __launch_bounds__(BLOCK) void flex_attn_merge_kernel(
     TlFlexExtra ex) {
   const int64_t row = blockIdx.x;
   const float* pr = part + row * ns * (2 + V);
-  float M = -INFINITY;
-  for (int z = 0; z < ns; ++z) M = fmaxf(M, pr[z * (2 + V)]);
+  // lane z of every wave holds split z's statistics (ns <= 64)
+  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+  const float mz = lane < ns ? pr[lane * (2 + V)] : -INFINITY;
+  const float lz = lane < ns ? pr[lane * (2 + V) + 1] : 0.f;
+  float M = wave_reduce_max(mz);
   const float sl = sinks ? sinks[row % H] : 0.f;
   if (sink) M = fmaxf(M, sl);
-  float L = sink ? expf(sl - M) : 0.f;
-  for (int z = 0; z < ns; ++z) {
-    const float mz = pr[z * (2 + V)];
-    L += (mz == -INFINITY ? 0.f : expf(mz - M)) * pr[z * (2 + V) + 1];
-  }
-  for (int c = threadIdx.x; c < V; c += BLOCK) {
+  const float wz = mz == -INFINITY ? 0.f : expf(mz - M);
+  const float L = wave_reduce_sum(wz * lz) + (sink ? expf(sl - M) : 0.f);
+  // whole waves walk the columns together: the weights come by shuffles
+  for (int c0 = threadIdx.x - lane; c0 < V; c0 += BLOCK) {
+    const int c = c0 + lane;
     float A = 0.f;
+#pragma unroll 8
     for (int z = 0; z < ns; ++z) {
-      const float mz = pr[z * (2 + V)];
-      A += (mz == -INFINITY ? 0.f : expf(mz - M)) * pr[z * (2 + V) + 2 + c];
+      const float w = __shfl(wz, z, WAVE_SIZE);
+      if (c < V) A += w * pr[z * (2 + V) + 2 + c];
     }
+    if (c >= V) continue;
     const float r = A / L * out_gate(ex, row / H, (int)(row % H), V, c);
     if (out_f32)
       ((float*)out)[row * V + c] = r;

@@ -89,6 +89,56 @@ __global__ __launch_bounds__(BLOCK) void route_logits_kernel(
     select_top(z, E, top, wt + t * top, idx + t * top);
 }
 
+// the same for W a multiple of 4: the token's row is staged in LDS and four
+// experts' rows are read side by side, 16 bytes at a time
+struct alignas(8) bf16x4 {
+  bf16 v[4];
+};
+DEVINLINE float4 ld4(const float* p) {
+  return *reinterpret_cast<const float4*>(p);
+}
+DEVINLINE float4 ld4(const bf16* p) {
+  const bf16x4 x = *reinterpret_cast<const bf16x4*>(p);
+  return make_float4(bf2f(x.v[0]), bf2f(x.v[1]), bf2f(x.v[2]), bf2f(x.v[3]));
+}
+
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void route_logits_vec_kernel(
+    const T* __restrict__ h, const float* __restrict__ w,
+    float* __restrict__ wt, int* __restrict__ idx, int W, int E, int top) {
+  extern __shared__ __align__(16) float sh[];       // hs[W] | z[E]
+  float* hs = sh;
+  float* z = sh + W;
+  const int64_t t = blockIdx.x;
+  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+  for (int c = threadIdx.x * 4; c < W; c += BLOCK * 4)
+    *reinterpret_cast<float4*>(hs + c) = ld4(h + t * W + c);
+  __syncthreads();
+  for (int e0 = (threadIdx.x / WAVE_SIZE) * 4; e0 < E; e0 += NWAVE * 4) {
+    const float* wr[4];
+    float s[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int u = 0; u < 4; ++u) wr[u] = w + (int64_t)min(e0 + u, E - 1) * W;
+#pragma unroll 4
+    for (int c = lane * 4; c < W; c += WAVE_SIZE * 4) {
+      const float4 x = *reinterpret_cast<const float4*>(hs + c);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const float4 y = ld4(wr[u] + c);
+        s[u] += x.x * y.x + x.y * y.y + x.z * y.z + x.w * y.w;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const float v = wave_reduce_sum(s[u]);
+      if (lane == 0 && e0 + u < E) z[e0 + u] = v;
+    }
+  }
+  __syncthreads();
+  if (threadIdx.x < WAVE_SIZE)
+    select_top(z, E, top, wt + t * top, idx + t * top);
+}
+
 // one wave per token, logits given
 __global__ __launch_bounds__(BLOCK) void route_select_kernel(
     const float* __restrict__ z, float* __restrict__ wt,
@@ -312,6 +362,18 @@ void tl_moe_route(const void* h, const void* w, const void* z, void* wt,
   }
   const size_t smem = sizeof(float) * E;
   dim3 grid((unsigned)T);
+  const size_t vmem = sizeof(float) * ((size_t)W + E);
+  if (W % 4 == 0 && vmem <= 48 * 1024) {
+    if (is_f32)
+      hipLaunchKernelGGL(route_logits_vec_kernel<float>, grid, block, vmem,
+                         stream, (const float*)h, (const float*)w, (float*)wt,
+                         (int*)idx, W, E, top);
+    else
+      hipLaunchKernelGGL(route_logits_vec_kernel<bf16>, grid, block, vmem,
+                         stream, (const bf16*)h, (const float*)w, (float*)wt,
+                         (int*)idx, W, E, top);
+    return;
+  }
   if (is_f32)
     hipLaunchKernelGGL(route_logits_kernel<float>, grid, block, smem, stream,
                        (const float*)h, (const float*)w, (float*)wt,

@@ -260,6 +260,64 @@ __global__ __launch_bounds__(BLOCK) void head_rms_gate_kernel(
   }
 }
 
+// the same for V a multiple of 4: LG lanes (a power of two) per (row, head),
+// four columns per lane and step
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void head_rms_gate_vec_kernel(
+    const float* __restrict__ x, const float* __restrict__ w,
+    const T* __restrict__ gate, int ldg, T* __restrict__ out, int64_t units,
+    int H, int V, float eps, int LG) {
+  const int64_t u = ((int64_t)blockIdx.x * BLOCK + threadIdx.x) / LG;
+  const bool on = u < units;      // a wave's lanes shuffle together
+  const int c0 = (threadIdx.x & (LG - 1)) * 4;
+  const float* xr = x + u * V;
+  float ss = 0.f;
+  if (on)
+    for (int c = c0; c < V; c += LG * 4) {
+      float v[4];
+      ld4(xr + c, v);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += v[e] * v[e];
+    }
+  for (int off = LG >> 1; off > 0; off >>= 1)
+    ss += __shfl_xor(ss, off, WAVE_SIZE);
+  if (!on) return;
+  const float rn = 1.0f / sqrtf(ss / (float)V + eps);
+  const T* gr = gate ? gate + (u / H) * ldg + (u % H) * V : nullptr;
+  for (int c = c0; c < V; c += LG * 4) {
+    float v[4], ww[4];
+    ld4(xr + c, v);
+    ld4(w + c, ww);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= rn * ww[e];
+    if (gate) {
+      float z[4];
+      ld4(gr + c, z);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] *= z[e] / (1.f + expf(-z[e]));
+    }
+    st4(out + u * V + c, v);
+  }
+}
+
+template <typename T>
+void launch_head_rms(const float* x, const float* w, const T* gate, int ldg,
+                     T* out, int64_t units, int H, int V, float eps, bool vec,
+                     hipStream_t stream) {
+  if (!vec) {
+    hipLaunchKernelGGL(head_rms_gate_kernel<T>,
+                       dim3((unsigned)((units + NW - 1) / NW)), dim3(BLOCK), 0,
+                       stream, x, w, gate, ldg, out, units, H, V, eps);
+    return;
+  }
+  int LG = 1;
+  while (LG < WAVE_SIZE && LG * 4 < V) LG <<= 1;
+  hipLaunchKernelGGL(head_rms_gate_vec_kernel<T>,
+                     dim3((unsigned)((units * LG + BLOCK - 1) / BLOCK)),
+                     dim3(BLOCK), 0, stream, x, w, gate, ldg, out, units, H, V,
+                     eps, LG);
+}
+
 // out = x / rms(x) * g [* sigmoid(gate)], x fp32 [rows, N]
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void rms_scale_kernel(
@@ -387,19 +445,18 @@ void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
 }
 
 void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
-                      void* out, int64_t rows, int H, int V, float eps,
-                      int is_f32, hipStream_t stream) {
+                      int gate_aligned, void* out, int64_t rows, int H, int V,
+                      float eps, int is_f32, hipStream_t stream) {
   const int64_t units = rows * H;
   if (units <= 0) return;
-  dim3 grid((unsigned)((units + NW - 1) / NW)), block(BLOCK);
+  const bool vec = V % 4 == 0 && (!gate || gate_aligned);
   if (is_f32)
-    hipLaunchKernelGGL(head_rms_gate_kernel<float>, grid, block, 0, stream,
-                       (const float*)x, (const float*)w, (const float*)gate,
-                       ldg, (float*)out, units, H, V, eps);
+    launch_head_rms<float>((const float*)x, (const float*)w,
+                           (const float*)gate, ldg, (float*)out, units, H, V,
+                           eps, vec, stream);
   else
-    hipLaunchKernelGGL(head_rms_gate_kernel<bf16>, grid, block, 0, stream,
-                       (const float*)x, (const float*)w, (const bf16*)gate,
-                       ldg, (bf16*)out, units, H, V, eps);
+    launch_head_rms<bf16>((const float*)x, (const float*)w, (const bf16*)gate,
+                          ldg, (bf16*)out, units, H, V, eps, vec, stream);
 }
 
 void tl_rms_scale(const void* x, const void* w, const void* gate, int ldg,

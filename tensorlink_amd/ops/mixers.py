@@ -1200,14 +1200,11 @@ def expert_gated_ff(h: torch.Tensor, wts: torch.Tensor, idx: torch.Tensor,
     products run in h's dtype with fp32 accumulation, the weighted sum is
     fp32; result in h's dtype."""
     T, W = h.shape
-    E, ff = gate_up.shape[0], gate_up.shape[1] // 2
-    top = idx.shape[1]
+    E = gate_up.shape[0]
     if h.is_cuda:
-        C = _ext()
-        seg, pair_tok, rank = C.moe_sort(idx, E)
-        a = C.moe_gemm_stacked(h.contiguous(), pair_tok, seg, gate_up)
-        y = C.moe_gemm_stacked(act_gate(a, act), None, seg, down)
-        return C.moe_combine(y, rank, wts, shared, sgate, int(sgate_col))
+        return _ext().moe_experts(h.contiguous(), wts, idx, gate_up, down,
+                                  GATE_ACTS[act], shared, sgate,
+                                  int(sgate_col))
     out = torch.zeros(T, W, dtype=torch.float32)
     for e in range(E):
         tok, choice = (idx == e).nonzero(as_tuple=True)
