@@ -125,6 +125,9 @@ class ModelConfig:
         if cfg.get("architecture") in ("Mogisun", "mogisun"):
             from tensorlink_amd.models.mogisun import MogisunConfig
             return MogisunConfig.from_dict(cfg, name=name)
+        if cfg.get("architecture") in ("Lunadra", "lunadra"):
+            from tensorlink_amd.models.lunadra import LunadraConfig
+            return LunadraConfig.from_dict(cfg, name=name)
         if "architecture" in cfg and "architectures" not in cfg:
             # our own to_json round-trip (save_hf_checkpoint writes it)
             known = {f.name for f in dataclasses.fields(cls)}

@@ -466,4 +466,7 @@ def _stage_class(config: ModelConfig):
     if config.architecture == "mogisun":
         from tensorlink_amd.models.mogisun import MogisunStageModel
         return MogisunStageModel
+    if config.architecture == "lunadra":
+        from tensorlink_amd.models.lunadra import LunadraStageModel
+        return LunadraStageModel
     return StageModel

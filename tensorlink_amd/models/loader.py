@@ -147,6 +147,11 @@ def load_stage_from_checkpoint(stage: StageModel, ckpt_dir: str,
         n = load_mogisun_weights(stage, ckpt_dir, dtype=dtype)
         stage.to(device=device, dtype=dtype)
         return n
+    if arch == "lunadra":
+        from tensorlink_amd.models.lunadra import load_lunadra_weights
+        n = load_lunadra_weights(stage, ckpt_dir, dtype=dtype)
+        stage.to(device=device, dtype=dtype)
+        return n
     from safetensors import safe_open
 
     index_path = os.path.join(ckpt_dir, "model.safetensors.index.json")
@@ -205,6 +210,10 @@ def init_random_stage(stage: StageModel, device="cpu", dtype=torch.bfloat16,
     if stage.config.architecture == "mogisun":
         from tensorlink_amd.models.mogisun import init_mogisun_random
         init_mogisun_random(stage, seed=seed)
+        return stage.to(device=device, dtype=dtype)
+    if stage.config.architecture == "lunadra":
+        from tensorlink_amd.models.lunadra import init_lunadra_random
+        init_lunadra_random(stage, seed=seed)
         return stage.to(device=device, dtype=dtype)
     gen_dev = device if str(device).startswith("cuda") else "cpu"
     g = torch.Generator(device=gen_dev)

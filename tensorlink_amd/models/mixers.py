@@ -42,6 +42,17 @@ class _F32Cache:
             store[name] = hit
         return hit[1]
 
+    def _f32_t(self, name: str) -> torch.Tensor:
+        """The same for a matrix, transposed."""
+        p = getattr(self, name)
+        store = self.__dict__.setdefault("_f32_t_store", {})
+        key = (p.data_ptr(), p._version, p.device, p.dtype)
+        hit = store.get(name)
+        if hit is None or hit[0] != key:
+            hit = (key, p.detach().float().t().contiguous())
+            store[name] = hit
+        return hit[1]
+
 
 class DynamicTanh(nn.Module, _F32Cache):
     """y = tanh(alpha * x) * weight + bias; no mean, no variance."""
@@ -70,26 +81,37 @@ class HyperConnection(nn.Module, _F32Cache):
 
 class MLSTMMixer(nn.Module, _F32Cache):
     """Matrix-memory mixer: fused q|k|v|g projection, fp32 soft-capped
-    gates, the slot-state recurrence kernel, output projection."""
+    gates, the slot-state recurrence kernel, output projection.
+
+    With ``hosted`` the projections belong to the caller (a layer whose
+    sublayers read one input): ``forward`` then takes the caller's projection
+    with ``in_cols`` columns [q | k | v | g] from ``col`` and the fp32 gate
+    pre-activations [input | forget] (bias added), the first ``thin_cols``
+    columns of ``thin``."""
 
     kind = "mlstm"
 
     def __init__(self, width: int, heads: int, dim: int, vdim: int,
-                 gate_cap: float, eps: float):
+                 gate_cap: float, eps: float, *, hosted: bool = False):
         super().__init__()
         self.H, self.D, self.V = heads, dim, vdim
         self.cap, self.eps = float(gate_cap), float(eps)
+        self.hosted = bool(hosted)
         hd, hv = heads * dim, heads * vdim
         self.offs = (0, hd, 2 * hd, 2 * hd + hv)
-        self.proj = TLLinear(width, 2 * hd + 2 * hv, bias=False)
-        self.gate = nn.Linear(width, 2 * heads, bias=True)   # input | forget
+        self.in_cols, self.thin_cols = 2 * hd + 2 * hv, 2 * heads
+        if not hosted:
+            self.proj = TLLinear(width, self.in_cols, bias=False)
+            self.gate = nn.Linear(width, 2 * heads, bias=True)  # input|forget
         self.norm = nn.Parameter(torch.ones(hv))
         self.o_proj = TLLinear(hv, width, bias=False)
 
     def cache_spec(self):
         return {"kind": "mlstm", "H": self.H, "D": self.D, "V": self.V}
 
-    def forward(self, h, meta, cache, layer_idx):
+    def forward(self, h, meta, cache, layer_idx, col: int = 0, thin=None):
+        if self.hosted:
+            return self._mix(h, col, thin, meta, cache.state[layer_idx])
         proj = self.proj(h)
         gw = self.gate.weight
         if gw.dtype != torch.float32:
@@ -102,9 +124,13 @@ class MLSTMMixer(nn.Module, _F32Cache):
             gates = F.linear(h.float(), store[1], store[2])
         else:
             gates = F.linear(h.float(), gw, self.gate.bias)
-        S, n, m = cache.state[layer_idx]
-        o = mx.mlstm_scan(proj, self.offs, gates, self._f32("norm"), S, n, m,
-                          meta, self.H, self.D, self.V, self.cap, self.eps)
+        return self._mix(proj, 0, gates, meta, cache.state[layer_idx])
+
+    def _mix(self, proj, col, gates, meta, state):
+        S, n, m = state
+        o = mx.mlstm_scan(proj, [c + col for c in self.offs], gates,
+                          self._f32("norm"), S, n, m, meta, self.H, self.D,
+                          self.V, self.cap, self.eps)
         return self.o_proj(o)
 
 
@@ -246,6 +272,12 @@ def pad_cols(n: int) -> int:
     """Rows of a fused projection rounded up to what the serving GEMM
     kernels take (a multiple of 64); the added rows are zero."""
     return (n + 63) // 64 * 64
+
+
+def align_cols(n: int) -> int:
+    """A column count rounded up so that what follows it in a fused
+    projection starts on a 16-byte boundary in bf16 and fp32."""
+    return (n + 7) // 8 * 8
 
 
 class RMSWeight(nn.Module, _F32Cache):
@@ -433,6 +465,10 @@ class WindowAttention(nn.Module, _F32Cache):
     ``side_cols``    this many further rows of the fused projection, with a
                      bias, belong to the caller: forward then returns
                      (output, projection, their first column);
+    ``hosted``       the input projection belongs to the caller: forward
+                     takes (projection, first column, ...) instead of the
+                     layer input, and ``in_cols`` columns [q | k | v | g]
+                     feed it;
     ``v_mix``        value mixing across layers: the first such layer of a
                      model publishes its values of the step's tokens in the
                      ``shared`` dictionary handed to forward, later ones
@@ -452,9 +488,11 @@ class WindowAttention(nn.Module, _F32Cache):
                  rel_far: float = 0.0, out_gate: bool = False,
                  v_mix: bool = False, unit_norm: bool = False,
                  q_temp: Optional[tuple] = None, head_gate: bool = False,
-                 bias: bool = False, side_cols: int = 0):
+                 bias: bool = False, side_cols: int = 0,
+                 hosted: bool = False):
         super().__init__()
         assert heads % kv_heads == 0 and rot_dims % 2 == 0 and rot_dims <= dim
+        assert not hosted or not (side_cols or v_mix)
         assert not (chunk and window), "a chunked mask has no window"
         assert not (unit_norm and qk_norm) and not (head_gate and out_gate)
         assert bias or not side_cols, "the caller's rows have a bias"
@@ -474,9 +512,10 @@ class WindowAttention(nn.Module, _F32Cache):
         self.side_col = self.q_cols + self.k_cols + self.v_cols
         self.g_col = self.side_col + self.side_cols
         self.g_cols = heads if head_gate else heads * vdim if out_gate else 0
-        cols = self.g_col + self.g_cols
-        self.qkv = TLLinear(width, pad_cols(cols) if side_cols else cols,
-                            bias=bias)
+        cols = self.in_cols = self.g_col + self.g_cols
+        self.hosted, self.state_shapes, self.thin_cols = bool(hosted), [], 0
+        self.qkv = None if hosted else TLLinear(
+            width, pad_cols(cols) if side_cols else cols, bias=bias)
         self.q_norm = nn.Parameter(torch.ones(
             dim if head_norm else self.q_cols)) if qk_norm else None
         self.k_norm = nn.Parameter(torch.ones(
@@ -515,17 +554,26 @@ class WindowAttention(nn.Module, _F32Cache):
             self.__dict__["_lut"] = hit
         return hit[1]
 
-    def forward(self, h, meta, cache, layer_idx, shared=None):
+    def forward(self, h, *args):
+        """(h, meta, cache, layer index, shared=None), or with ``hosted``
+        (projection, column, meta, key pool, value pool)."""
+        if self.hosted:
+            return self._attend(h, *args)
+        meta, cache, layer_idx = args[:3]
         proj = self.qkv(h)
-        fr = self._freqs(h.device) if self.rot_dims else None
+        y = self._attend(proj, 0, meta, cache.k[layer_idx],
+                         cache.v[layer_idx], *args[3:])
+        return (y, proj, self.side_col) if self.side_cols else y
+
+    def _attend(self, proj, col, meta, kpool, vpool, shared=None):
+        fr = self._freqs(proj.device) if self.rot_dims else None
         qn = self._f32("q_norm") if self.q_norm is not None else None
         kn = self._f32("k_norm") if self.k_norm is not None else None
-        kpool, vpool = cache.k[layer_idx], cache.v[layer_idx]
-        v_col = self.q_cols + self.k_cols
+        v_col = col + self.q_cols + self.k_cols
         rot = dict(rot_dims=self.rot_dims, freqs=fr,
                    interleaved=self.interleaved,
                    head_norm=self.head_norm or self.unit_norm, eps=self.eps)
-        mx.norm_rope_rows(proj, self.q_cols, self.G, self.D, meta,
+        mx.norm_rope_rows(proj, col + self.q_cols, self.G, self.D, meta,
                           norm_w=kn, norm_cols=self.k_cols, pool=kpool, **rot)
         first = None
         if self.v_mix:
@@ -544,7 +592,7 @@ class WindowAttention(nn.Module, _F32Cache):
             mx.norm_rope_rows(proj, v_col, self.G, self.V, meta, pool=vpool,
                               mix_src=first[0], mix_col=first[1],
                               mix_lam=self._f32("vmix").reshape(1))
-        q = mx.norm_rope_rows(proj, 0, self.H, self.D, meta, norm_w=qn,
+        q = mx.norm_rope_rows(proj, col, self.H, self.D, meta, norm_w=qn,
                               norm_cols=self.q_cols, temp=self.q_temp, **rot)
         o = mx.flex_attention(
             q, kpool, vpool, meta, self.H, self.scale, window=self.window,
@@ -553,12 +601,10 @@ class WindowAttention(nn.Module, _F32Cache):
             sink_logits=self._f32("sinks") if self.sinks is not None
             else None,
             chunk=self.chunk, keep_first=self.keep_first,
-            dist_bias=self._dist_bias(h.device) if self.rel is not None
+            dist_bias=self._dist_bias(proj.device) if self.rel is not None
             else None,
-            gate=proj if self.g_cols else None, gate_col=self.g_col,
-            gate_heads=self.head_gate, out_dtype=h.dtype)
-        if self.side_cols:
-            return self.o_proj(o), proj, self.side_col
+            gate=proj if self.g_cols else None, gate_col=col + self.g_col,
+            gate_heads=self.head_gate, out_dtype=proj.dtype)
         return self.o_proj(o)
 
 
@@ -577,25 +623,31 @@ class DenseFF(nn.Module):
 
 class GatedFF(nn.Module):
     """down(act(gate x) * (up x)), no biases; ``act`` is the tanh-form or
-    exact GELU (``tanh_form``) or "silu"; gate and up are one fused
-    projection [gate | up]. ``side_cols`` further rows of it, with a bias,
-    belong to the caller: forward then returns (output, projection, their
-    first column)."""
+    exact GELU (``tanh_form``) or what ``ops.mixers.act_gate`` takes; gate
+    and up are one fused projection [gate | up]. ``side_cols`` further rows
+    of it, with a bias, belong to the caller: forward then returns (output,
+    projection, their first column). With ``hosted`` the projection itself
+    is the caller's: forward takes it and the first of its ``in_cols``
+    columns."""
 
     kind = "dense"
 
     def __init__(self, width: int, ff: int, tanh_form: bool = True, *,
-                 act: Optional[str] = None, side_cols: int = 0):
+                 act=None, side_cols: int = 0, hosted: bool = False):
         super().__init__()
+        assert not (hosted and side_cols)
+        self.hosted, self.in_cols, self.thin_cols = bool(hosted), 2 * ff, 0
         self.ff, self.side_cols = int(ff), int(side_cols)
         self.act = act or ("gelu_tanh" if tanh_form else "gelu")
         self.side_col = 2 * self.ff
-        self.gate_up = TLLinear(
+        self.gate_up = None if hosted else TLLinear(
             width, pad_cols(2 * ff + side_cols) if side_cols else 2 * ff,
             bias=bool(side_cols))
         self.down = TLLinear(ff, width, bias=False)
 
-    def forward(self, h):
+    def forward(self, h, col: int = 0):
+        if self.hosted:
+            return self.down(mx.act_gate(h, self.act, self.ff, col))
         p = self.gate_up(h)
         y = self.down(mx.act_gate(p, self.act, self.ff))
         return (y, p, self.side_col) if self.side_cols else y
@@ -762,30 +814,49 @@ class SSDMixer(nn.Module, _F32Cache):
 
 class ParallelMixer(nn.Module, _F32Cache):
     """A pair of mixers fed by the same input: ``left`` (attention) and
-    ``right`` (state-space), fed by ONE fused input projection. The result
-    is half the sum of the two outputs after each is RMS-normed over the
-    model width with its plain weight (``left_out`` / ``right_out``);
-    ``forward`` returns the two raw outputs and the caller's residual
-    update applies the norms and the half sum in the same pass."""
+    ``right`` (a recurrence), fed by ONE fused input projection. By default
+    the result is half the sum of the two outputs after each is RMS-normed
+    over the model width with its plain weight (``left_out`` /
+    ``right_out``); with ``scales`` = (left, right) it is the plain weighted
+    sum. ``forward`` returns the two raw outputs; the caller's residual
+    update applies the norms, or the factors, in the same pass.
+
+    With ``hosted`` (needs ``scales``) the projection is the caller's too:
+    forward takes it, the first of its ``in_cols`` columns, and the caller's
+    fp32 columns ``thin`` when the right mixer has ``thin_cols``."""
 
     kind = "parallel"
 
-    def __init__(self, width: int, left: nn.Module, right: nn.Module):
+    def __init__(self, width: int, left: nn.Module, right: nn.Module, *,
+                 scales: Optional[tuple] = None, hosted: bool = False):
         super().__init__()
+        assert not hosted or scales is not None
         self.left, self.right = left, right
-        self.proj = TLLinear(width, left.in_cols + right.in_cols, bias=True)
-        self.left_out = nn.Parameter(torch.ones(width))
-        self.right_out = nn.Parameter(torch.ones(width))
+        self.hosted = bool(hosted)
+        self.scales = tuple(float(x) for x in scales) if scales else None
+        # the right mixer's columns start on a 16-byte boundary
+        self.right_col = (align_cols(left.in_cols) if hosted
+                          else left.in_cols)
+        self.in_cols = self.right_col + right.in_cols
+        self.thin_cols = getattr(right, "thin_cols", 0)
+        self.proj = None if hosted else TLLinear(width, self.in_cols,
+                                                 bias=True)
+        if scales is None:
+            self.left_out = nn.Parameter(torch.ones(width))
+            self.right_out = nn.Parameter(torch.ones(width))
         self.state_shapes = list(left.state_shapes) + list(right.state_shapes)
 
     def cache_spec(self):
         return dict(self.left.cache_spec(), shapes=self.state_shapes)
 
-    def forward(self, h, meta, kpool, vpool, states):
-        proj = self.proj(h)
+    def forward(self, h, meta, kpool, vpool, states, col: int = 0,
+                thin=None):
+        proj = h if self.hosted else self.proj(h)
         nl = len(self.left.state_shapes)
-        a = self.left(proj, 0, meta, kpool, vpool, *states[:nl])
-        b = self.right(proj, self.left.in_cols, meta, *states[nl:])
+        a = self.left(proj, col, meta, kpool, vpool, *states[:nl])
+        extra = (thin,) if self.thin_cols else ()
+        b = self.right(proj, col + self.right_col, meta, *states[nl:],
+                       *extra)
         return a, b
 
 
@@ -843,20 +914,10 @@ class GatedLinearAttention(nn.Module, _F32Cache):
     def cache_spec(self):
         return {"kind": "state", "shapes": [(self.H, self.D, self.V)]}
 
-    def _a2t(self):
-        """a2 transposed, fp32 [rank, heads*dim]; rebuilt when it changes."""
-        p = self.a2
-        key = (p.data_ptr(), p._version, p.device, p.dtype)
-        hit = self.__dict__.get("_a2t_hit")
-        if hit is None or hit[0] != key:
-            hit = (key, p.detach().float().t().contiguous())
-            self.__dict__["_a2t_hit"] = hit
-        return hit[1]
-
     def forward(self, h, meta, cache, layer_idx, shared=None):
         proj = self.proj(h)
         (S,) = cache.state[layer_idx]
-        o = mx.gla_scan(proj, self.offs + (self.a_col,), self._a2t(),
+        o = mx.gla_scan(proj, self.offs + (self.a_col,), self._f32_t("a2"),
                         self._f32("a2_b"), self.tau, S, meta, self.H, self.D,
                         self.V)
         y = mx.rms_scale(o, self._f32("norm"), self.eps, False, gate=proj,
@@ -867,44 +928,141 @@ class GatedLinearAttention(nn.Module, _F32Cache):
 
 
 class GatedMoE(nn.Module, _F32Cache):
-    """Mixture of gated experts down(act(gate x) * (up x)), no biases:
-    fp32 router, the ``top`` largest logits chosen and weighted by the
-    softmax over the chosen ones; optionally a shared expert of the same
-    form (``shared_ff`` > 0) for every token, times sigmoid of one more
-    projection of the input.
+    """Mixture of gated experts down(act(gate x) * (up x)), no biases
+    (``act``: what ``ops.mixers.act_gate`` takes), behind an fp32 router;
+    optionally a shared expert of the same form (``shared_ff`` > 0) for
+    every token, times sigmoid of one more projection of the input.
 
     The dense rows — the shared expert's gate and up, its sigmoid's row and
     the caller's ``side_cols`` (with a bias) — are one fused projection
     [gate | up | side | sg]; the routed experts are stacked and run as
-    grouped products over expert-sorted (token, choice) pairs."""
+    grouped products over expert-sorted (token, choice) pairs.
+
+    Options:
+    ``scores``     by default the ``top`` largest logits are chosen and
+                   weighted by the softmax over the chosen ones; with
+                   ``scores`` the softmax runs over all experts, a learned
+                   ``correction`` per expert is added for the choice only,
+                   and the chosen experts' scores are the weights;
+    ``identity``   this many further router outputs, after the experts', are
+                   experts that return their input (needs ``scores``);
+    ``shared_act`` the shared expert's activation, if not ``act``;
+    ``shared_gate``  False: the shared expert is added as it is;
+    ``hosted``     the input projections belong to the caller: ``in_cols``
+                   columns [gate | up] of the shared expert from ``col`` of
+                   its projection ``proj`` and ``thin_cols`` fp32 router
+                   logits from column ``tcol`` of ``thin`` (needs
+                   ``scores``, no ``shared_gate``)."""
 
     kind = "moe"
 
     def __init__(self, width: int, ff: int, experts: int, top: int,
-                 shared_ff: int = 0, *, act: str = "silu",
-                 side_cols: int = 0):
+                 shared_ff: int = 0, *, act="silu", side_cols: int = 0,
+                 scores: bool = False, identity: int = 0, shared_act=None,
+                 shared_gate: bool = True, hosted: bool = False):
         super().__init__()
-        assert 1 <= top <= experts
+        assert 1 <= top <= experts + identity
+        assert scores or not (identity or hosted)
+        assert not hosted or not (side_cols or (shared_ff and shared_gate))
         self.W, self.ff, self.E, self.top = width, int(ff), experts, int(top)
         self.sff, self.act = int(shared_ff), act
+        self.shared_act = shared_act or act
+        self.shared_gate = bool(shared_gate)
+        self.scores, self.identity = bool(scores), int(identity)
+        self.hosted, self.in_cols = bool(hosted), 2 * self.sff
+        self.thin_cols = experts + self.identity if hosted else 0
         self.side_cols, self.side_col = int(side_cols), 2 * self.sff
         self.sg_col = self.side_col + self.side_cols
-        self.router = nn.Parameter(torch.zeros(experts, width))
+        self.router = None if hosted else nn.Parameter(
+            torch.zeros(experts + self.identity, width))
+        self.correction = nn.Parameter(
+            torch.zeros(experts + self.identity)) if scores else None
         self.gate_up = nn.Parameter(torch.zeros(experts, 2 * self.ff, width))
         self.down = nn.Parameter(torch.zeros(experts, width, self.ff))
-        cols = self.sg_col + (1 if self.sff else 0)
+        cols = self.sg_col + (1 if self.sff and shared_gate else 0)
         self.dense = TLLinear(width, pad_cols(cols), bias=bool(side_cols)) \
-            if cols else None
+            if cols and not hosted else None
         self.shared_down = TLLinear(self.sff, width, bias=False) \
             if self.sff else None
 
-    def forward(self, h):
-        wts, idx = mx.topk_softmax_router(h, self._f32("router"), self.top)
-        p = self.dense(h) if self.dense is not None else None
-        s = (self.shared_down(mx.act_gate(p, self.act, self.sff))
+    def forward(self, h, proj=None, col: int = 0, thin=None, tcol: int = 0):
+        p = proj
+        if not self.hosted and self.dense is not None:
+            p = self.dense(h)
+        if self.scores:
+            if not self.hosted:
+                thin, tcol = mx.thin_linear(h, self.router), 0
+            wts, idx = mx.score_router(thin, tcol, self.E + self.identity,
+                                       self._f32("correction"), self.top)
+        else:
+            wts, idx = mx.topk_softmax_router(h, self._f32("router"),
+                                              self.top)
+        s = (self.shared_down(mx.act_gate(p, self.shared_act, self.sff, col))
              if self.sff else None)
-        y = mx.expert_gated_ff(h, wts, idx, self.gate_up, self.down,
-                               self.act, shared=s,
-                               sgate=p if self.sff else None,
-                               sgate_col=self.sg_col)
+        y = mx.expert_gated_ff(
+            h, wts, idx, self.gate_up, self.down, self.act, shared=s,
+            sgate=p if self.sff and self.shared_gate else None,
+            sgate_col=self.sg_col, identity=self.identity)
         return (y, p, self.side_col) if self.side_cols else y
+
+
+# ---------------------------------------------------------------------------
+# gated delta rule
+# ---------------------------------------------------------------------------
+class GatedDeltaMixer(nn.Module, _F32Cache):
+    """Gated delta rule: a linear-attention memory that corrects what a key
+    already reads before it writes, with one decay per key channel and
+    token. q, k (``kv_heads`` x dim) and v (heads x vdim) pass a short causal
+    convolution and silu; q and k become unit vectors; then, per head,
+    S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q (see
+    ``ops.mixers.delta_scan``). Every head's read-out is RMS-normed over
+    vdim with one shared weight, times sigmoid of a low-rank projection
+    g2 (g1 x), then the output projection.
+
+    The input projections belong to the caller: ``in_cols`` columns
+    [q | k | v | a1 | g1] of its projection from ``col``, and ``thin_cols``
+    fp32 columns (raw beta) of ``thin``. Per-sequence memory: the
+    convolution's last inputs and the fp32 state [heads, dim, vdim]."""
+
+    kind = "gated_delta"
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, conv: int, decay_rank: int, gate_rank: int,
+                 eps: float):
+        super().__init__()
+        assert heads % kv_heads == 0
+        self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
+        self.K, self.eps = int(conv), float(eps)
+        qk, hv = kv_heads * dim, heads * vdim
+        self.offs = (0, qk, 2 * qk)                      # q | k | v
+        self.conv_cols = 2 * qk + hv
+        self.R, self.GR = int(decay_rank), int(gate_rank)
+        self.a_col = align_cols(self.conv_cols)
+        self.g_col = align_cols(self.a_col + self.R)
+        self.in_cols, self.thin_cols = self.g_col + self.GR, heads
+        self.conv = nn.Parameter(torch.zeros(self.conv_cols, self.K))
+        self.A_log = nn.Parameter(torch.zeros(heads))
+        self.a2 = nn.Parameter(torch.zeros(heads * dim, self.R))
+        self.dt_bias = nn.Parameter(torch.zeros(heads * dim))
+        self.g2 = nn.Parameter(torch.zeros(hv, self.GR))
+        self.norm = nn.Parameter(torch.ones(vdim))
+        self.o_proj = TLLinear(hv, width, bias=False)
+        self.state_shapes = [(self.K - 1, self.conv_cols),
+                             (heads, dim, vdim)]
+
+    def cache_spec(self):
+        return {"kind": "state", "shapes": self.state_shapes}
+
+    def forward(self, proj, col, meta, hist, S, thin):
+        x = mx.conv_rope_rows(proj, col, 1, self.conv_cols,
+                              self._f32("conv"), hist, meta, silu=True)
+        o = mx.delta_scan(x, self.offs, proj, col + self.a_col, thin, 0,
+                          self._f32_t("a2"), self._f32("dt_bias"),
+                          self._f32("A_log"), S, meta, self.H, self.G, self.D,
+                          self.V)
+        c = col + self.g_col
+        gate = F.linear(proj[:, c:c + self.GR], self.g2)
+        y = mx.rms_scale(o, self._f32("norm"), self.eps, False, gate=gate,
+                         out_dtype=proj.dtype, heads=self.H,
+                         gate_act="sigmoid")
+        return self.o_proj(y)

@@ -158,11 +158,14 @@ class HybridSlotCache(DynamicPagedKVCache):
     rows only, for layers whose values are part of the key row; an optional
     ``"shapes"`` list adds fp32 per-slot state tensors beside the pools),
     ``{"kind": "kv_ref", "src": j}``, ``{"kind": "mlstm", "H", "D",
-    "V"}`` or ``{"kind": "state", "shapes": [...]}``. ``k[l]`` / ``v[l]``
+    "V"}``, ``{"kind": "state", "shapes": [...]}`` or ``{"kind":
+    "last_token"}`` (the id of a sequence's last token, int32 [slots], for
+    embeddings that look back). ``k[l]`` / ``v[l]``
     are [pool_pages, G, PAGE, DK|V] (None for recurrent layers, the
     source's tensors for references); ``state[l]`` is (S [slots, H, D, V],
     n [slots, H, D], m [slots, H]) for ``mlstm``, one fp32 tensor
-    [slots, *shape] per entry of ``shapes`` for ``state``, else None. Pages
+    [slots, *shape] per entry of ``shapes`` for ``state``, the one int32
+    tensor for ``last_token``, else None. Pages
     are leased and returned exactly as in :class:`DynamicPagedKVCache`;
     recurrent state needs no clearing on release because the kernels start
     a sequence with no cached tokens from zeros."""
@@ -198,6 +201,11 @@ class HybridSlotCache(DynamicPagedKVCache):
                     torch.zeros(slots, *shape, device=device,
                                 dtype=torch.float32)
                     for shape in sp["shapes"]))
+            elif sp["kind"] == "last_token":
+                self.k.append(None)
+                self.v.append(None)
+                self.state.append((torch.zeros(slots, device=device,
+                                               dtype=torch.int32),))
             else:
                 f32 = dict(device=device, dtype=torch.float32)
                 self.k.append(None)

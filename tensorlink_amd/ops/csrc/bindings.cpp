@@ -494,12 +494,14 @@ void register_mix_ops(pybind11::module& mod);  // bindings_mix.cpp
 void register_seq_ops(pybind11::module& mod);  // bindings_seq.cpp
 void register_ssm_ops(pybind11::module& mod);  // bindings_ssm.cpp
 void register_gla_ops(pybind11::module& mod);  // bindings_gla.cpp
+void register_delta_ops(pybind11::module& mod);  // bindings_delta.cpp
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, mod) {
   register_mix_ops(mod);
   register_seq_ops(mod);
   register_ssm_ops(mod);
   register_gla_ops(mod);
+  register_delta_ops(mod);
   mod.def("rope_append_", &rope_append_,
           "fused RoPE + KV-cache append from fused-QKV rows");
   mod.def("swiglu_fused", &swiglu_fused, "silu-mul on fused [.,2I] rows");

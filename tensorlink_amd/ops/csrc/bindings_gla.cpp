@@ -26,6 +26,9 @@ int tl_moe_max_top();
 void tl_moe_route(const void* h, const void* w, const void* z, void* wt,
                   void* idx, int64_t T, int W, int E, int top, int is_f32,
                   hipStream_t stream);
+void tl_moe_route_scores(const void* z, int64_t ldz, const void* corr,
+                         void* wt, void* idx, int64_t T, int E, int top,
+                         hipStream_t stream);
 int tl_moe_sort_blocks(int P);
 void tl_moe_sort(const void* idx, int P, int E, int top, void* seg,
                  void* pair_tok, void* rank, void* hist, hipStream_t stream);
@@ -42,11 +45,12 @@ void tl_moe_rows(const void* x, const void* tok, const void* seg,
                  const void* w, void* out, int P, int E, int N, int K,
                  hipStream_t stream);
 void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
-                 int64_t rows, int N, int act, int is_f32,
-                 hipStream_t stream);
+                 int64_t rows, int N, int act, float lim, float alpha,
+                 int is_f32, hipStream_t stream);
 void tl_moe_combine(const void* y, const void* rank, const void* wt,
                     const void* shared, const void* sg, int ldg, int sg_col,
-                    void* out, int64_t T, int W, int top, int is_f32,
+                    const void* ident, const void* n_real, void* out,
+                    int64_t T, int W, int top, int is_f32,
                     hipStream_t stream);
 }
 
@@ -187,6 +191,31 @@ std::vector<Tensor> moe_route(Tensor h, Tensor w, c10::optional<Tensor> z,
   return {wt, idx};
 }
 
+// fp32 logits z[:, col:col + E]: scores = softmax over all E, the `top`
+// largest of score + corr chosen, weighted by their scores
+std::vector<Tensor> moe_route_scores(Tensor z, int64_t col, int64_t E,
+                                     c10::optional<Tensor> corr,
+                                     int64_t top) {
+  GLA_F32(z);
+  TORCH_CHECK(z.dim() == 2 && col >= 0 && E >= 1 && col + E <= z.size(1),
+              "logit columns out of range");
+  TORCH_CHECK(top >= 1 && top <= E && top <= tl_moe_max_top() &&
+                  E <= tl_moe_max_experts(),
+              "router sizes outside the kernel's range");
+  if (corr.has_value()) {
+    GLA_F32(corr.value());
+    TORCH_CHECK(corr->numel() == E, "one correction per expert");
+  }
+  const int64_t T = z.size(0);
+  auto wt = torch::empty({T, top}, z.options());
+  auto idx = torch::empty({T, top}, z.options().dtype(torch::kInt));
+  tl_moe_route_scores((const float*)z.data_ptr() + col, z.size(1),
+                      corr.has_value() ? corr->data_ptr() : nullptr,
+                      wt.data_ptr(), idx.data_ptr(), T, (int)E, (int)top,
+                      gla_stream());
+  return {wt, idx};
+}
+
 // idx [T, top] int32 in [0, E): (segments [E + 1], token of every sorted
 // pair [P], sorted position of every pair [T, top])
 std::vector<Tensor> moe_sort(Tensor idx, int64_t E) {
@@ -245,10 +274,13 @@ Tensor moe_gemm_stacked(Tensor x, c10::optional<Tensor> tok, Tensor seg,
   return out;
 }
 
-// sum_j wt[t][j] y[rank[t][j]] (+ sigmoid(sg[t][sg_col]) * shared[t])
+// sum_j wt[t][j] y[rank[t][j]] (+ sigmoid(sg[t][sg_col]) * shared[t]); with
+// `ident` pairs at sorted positions >= n_real[0] stand for the token's row of
+// it
 Tensor moe_combine(Tensor y, Tensor rank, Tensor wt,
                    c10::optional<Tensor> shared, c10::optional<Tensor> sg,
-                   int64_t sg_col) {
+                   int64_t sg_col, c10::optional<Tensor> ident,
+                   c10::optional<Tensor> n_real) {
   GLA_IN(y);
   GLA_I32(rank);
   GLA_F32(wt);
@@ -272,35 +304,57 @@ Tensor moe_combine(Tensor y, Tensor rank, Tensor wt,
       ldg = (int)sg->size(1);
     }
   }
+  if (ident.has_value()) {
+    GLA_IN(ident.value());
+    TORCH_CHECK(n_real.has_value() && ident->dim() == 2 &&
+                    ident->size(0) == T && ident->size(1) == W &&
+                    ident->scalar_type() == y.scalar_type(),
+                "identity rows must be [T, W]");
+    GLA_I32(n_real.value());
+  }
   auto out = torch::empty({T, W}, y.options());
   tl_moe_combine(y.data_ptr(), rank.data_ptr(), wt.data_ptr(),
                  shared.has_value() ? shared->data_ptr() : nullptr,
                  shared.has_value() && sg.has_value() ? sg->data_ptr()
                                                       : nullptr,
-                 ldg, (int)sg_col, out.data_ptr(), T, (int)W,
-                 (int)rank.size(1), gla_is_f32(y), gla_stream());
+                 ldg, (int)sg_col,
+                 ident.has_value() ? ident->data_ptr() : nullptr,
+                 ident.has_value() ? n_real->data_ptr() : nullptr,
+                 out.data_ptr(), T, (int)W, (int)rank.size(1), gla_is_f32(y), gla_stream());
   return out;
 }
 
 // the routed experts of a step in one call: sort, gate|up product,
-// activation, down product, combine (gate_up [E, 2 ff, W], down [E, W, ff])
+// activation, down product, combine (gate_up [E, 2 ff, W], down [E, W, ff]).
+// Indices E .. E + identity - 1 are identity experts: their pairs sort behind
+// the others, no product reads them, and the combine adds the token's h.
 Tensor moe_experts(Tensor h, Tensor wt, Tensor idx, Tensor gate_up,
-                   Tensor down, int64_t act, c10::optional<Tensor> shared,
+                   Tensor down, int64_t act, double lim, double alpha,
+                   int64_t identity, c10::optional<Tensor> shared,
                    c10::optional<Tensor> sg, int64_t sg_col) {
   TORCH_CHECK(gate_up.dim() == 3 && down.dim() == 3 && h.dim() == 2 &&
                   gate_up.size(1) == 2 * down.size(2) &&
                   gate_up.size(0) == down.size(0) &&
                   down.size(1) == h.size(1) && idx.dim() == 2 &&
-                  idx.size(0) == h.size(0) && act >= 0 && act <= 2,
+                  idx.size(0) == h.size(0) && act >= 0 && act <= 4 &&
+                  identity >= 0,
               "h [T, W], idx [T, top], gate_up [E, 2 ff, W], down [E, W, ff]");
-  auto s = moe_sort(idx, gate_up.size(0));
-  Tensor a = moe_gemm_stacked(h, s[1], s[0], gate_up);
+  const int64_t E = gate_up.size(0);
+  auto s = moe_sort(idx, E + identity);
+  Tensor seg = s[0].narrow(0, 0, E + 1);
+  Tensor a = moe_gemm_stacked(h, s[1], seg, gate_up);
   const int64_t ff = down.size(2);
   auto b = torch::empty({a.size(0), ff}, a.options());
   tl_act_gate(a.data_ptr(), 2 * ff, ff % 8 == 0, b.data_ptr(), a.size(0),
-              (int)ff, (int)act, gla_is_f32(a), gla_stream());
-  Tensor y = moe_gemm_stacked(b, c10::nullopt, s[0], down);
-  return moe_combine(y, s[2], wt, shared, sg, sg_col);
+              (int)ff, (int)act, (float)lim, (float)alpha, gla_is_f32(a),
+              gla_stream());
+  Tensor y = moe_gemm_stacked(b, c10::nullopt, seg, down);
+  c10::optional<Tensor> ident, n_real;
+  if (identity > 0) {
+    ident = h;
+    n_real = s[0].narrow(0, E, 1);
+  }
+  return moe_combine(y, s[2], wt, shared, sg, sg_col, ident, n_real);
 }
 
 }  // namespace
@@ -314,6 +368,8 @@ void register_gla_ops(pybind11::module& mod) {
           "gated linear attention, chunk form on fp32 MFMA");
   mod.def("moe_route", &moe_route,
           "top-k router with the softmax over the chosen logits");
+  mod.def("moe_route_scores", &moe_route_scores,
+          "top-k router on corrected softmax scores, logits given");
   mod.def("moe_sort", &moe_sort, "expert-sorted (token, choice) pairs");
   mod.def("moe_gemm_stacked", &moe_gemm_stacked,
           "grouped product with stacked experts, any size, bf16 or fp32");

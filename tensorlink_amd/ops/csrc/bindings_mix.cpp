@@ -16,8 +16,8 @@ void tl_hyper_dyt(void* X, const void* y, const void* mix, const void* outw,
 void tl_relu_sq(const void* x, void* out, int64_t n, int is_f32,
                 hipStream_t stream);
 int tl_mlstm_seq(const void* proj, int ld, int q_off, int k_off, int v_off,
-                 int g_off, const void* gates, const void* norm_w, void* S,
-                 void* n, void* m, const void* cu, const void* slots,
+                 int g_off, const void* gates, int ldg, const void* norm_w,
+                 void* S, void* n, void* m, const void* cu, const void* slots,
                  const void* pos0, void* out, int B, int H, int D, int V,
                  float cap, float qscale, float eps, void* F, int summary,
                  int is_f32, hipStream_t stream);
@@ -156,7 +156,9 @@ Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
   TORCH_CHECK(q_off + H * D <= ld && k_off + H * D <= ld &&
                   v_off + H * V <= ld && g_off + H * V <= ld,
               "projection columns out of range");
-  TORCH_CHECK(gates.numel() == T * 2 * H, "gates must be [T, 2H]");
+  TORCH_CHECK(gates.dim() == 2 && gates.size(0) == T &&
+                  gates.size(1) >= 2 * H,
+              "gates must be [T, >= 2H]");
   TORCH_CHECK(norm_w.numel() == H * V, "norm weight must be [H*V]");
   TORCH_CHECK(S.dim() == 4 && S.size(1) == H && S.size(2) == D &&
                   S.size(3) == V,
@@ -172,7 +174,8 @@ Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
   if (T == 0 || B == 0) return out;
   const int rc = tl_mlstm_seq(
       proj.data_ptr(), (int)ld, (int)q_off, (int)k_off, (int)v_off,
-      (int)g_off, gates.data_ptr(), norm_w.data_ptr(), S.data_ptr(),
+      (int)g_off, gates.data_ptr(), (int)gates.size(1), norm_w.data_ptr(),
+      S.data_ptr(),
       n.data_ptr(), m.data_ptr(), cu.data_ptr(), slots.data_ptr(),
       pos0.data_ptr(), out.data_ptr(), B, (int)H, (int)D, (int)V, (float)cap,
       (float)qscale, (float)eps, summary ? F_sum->data_ptr() : nullptr,

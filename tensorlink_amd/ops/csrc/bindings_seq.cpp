@@ -20,13 +20,14 @@ void tl_rms_scale(const void* x, const void* w, const void* gate, int ldg,
                   int one_plus, int is_f32, hipStream_t stream);
 void tl_add_rms(void* X, const void* y, const void* w, void* h, int64_t rows,
                 int W, float eps, float x_scale, const void* gate, int ldg,
-                int gate_aligned, int is_f32, hipStream_t stream);
+                int gate_aligned, float s0, const void* y1, float s1,
+                const void* y2, float s2, int is_f32, hipStream_t stream);
 void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
-                 int64_t rows, int N, int act, int is_f32,
-                 hipStream_t stream);
+                 int64_t rows, int N, int act, float lim, float alpha,
+                 int is_f32, hipStream_t stream);
 void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
                       int gate_aligned, void* out, int64_t rows, int H, int V,
-                      float eps, int is_f32, hipStream_t stream);
+                      float eps, int sig, int is_f32, hipStream_t stream);
 void tl_gelu(const void* x, void* out, int64_t n, int N, int tanh_form,
              const void* table, int ldt, int table_col, const void* tokens,
              int is_f32, hipStream_t stream);
@@ -146,11 +147,14 @@ Tensor rms_scale(Tensor x, Tensor w, double eps, bool one_plus,
   return out;
 }
 
-// X (*= x_scale) += y [* sigmoid(gate columns)]; returns rms(X) * w in the
-// serving dtype, or, without a weight, X itself after the add
+// X (*= x_scale) += s0 y [* sigmoid(gate columns)] + s1 y1 + s2 y2; returns
+// rms(X) * w in the serving dtype, or, without a weight, X itself after the
+// add
 Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
                double eps, double x_scale, c10::optional<Tensor> gate,
-               int64_t gate_col, bool out_f32) {
+               int64_t gate_col, double s0, c10::optional<Tensor> y1,
+               double s1, c10::optional<Tensor> y2, double s2,
+               bool out_f32) {
   SEQ_F32(X);
   TORCH_CHECK(X.dim() == 2, "X must be [T, W]");
   if (w.has_value()) {
@@ -162,6 +166,13 @@ Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
     TORCH_CHECK(y->sizes() == X.sizes(), "y must be [T, W]");
     TORCH_CHECK(act_is_f32(y.value()) == (out_f32 ? 1 : 0),
                 "y / output dtype mismatch");
+  }
+  for (const auto* m : {&y1, &y2}) {
+    if (!m->has_value()) continue;
+    SEQ_IN(m->value());
+    TORCH_CHECK(y.has_value() && m->value().sizes() == X.sizes() &&
+                    m->value().scalar_type() == y->scalar_type(),
+                "further terms must be [T, W] of y's dtype, beside y");
   }
   const char* gp = nullptr;
   int ldg = 0, gate_aligned = 0;
@@ -182,28 +193,33 @@ Tensor add_rms(Tensor X, c10::optional<Tensor> y, c10::optional<Tensor> w,
   tl_add_rms(X.data_ptr(), y.has_value() ? y->data_ptr() : nullptr,
              w.has_value() ? w->data_ptr() : nullptr,
              w.has_value() ? h.data_ptr() : nullptr, X.size(0), (int)X.size(1),
-             (float)eps, (float)x_scale, gp, ldg, gate_aligned,
+             (float)eps, (float)x_scale, gp, ldg, gate_aligned, (float)s0,
+             y1.has_value() ? y1->data_ptr() : nullptr, (float)s1,
+             y2.has_value() ? y2->data_ptr() : nullptr, (float)s2,
              out_f32 ? 1 : 0, seq_stream());
   return h;
 }
 
 // act(p[:, col:col + N]) * p[:, col + N:col + 2N]
-Tensor act_gate(Tensor p, int64_t col, int64_t N, int64_t act) {
+Tensor act_gate(Tensor p, int64_t col, int64_t N, int64_t act, double lim,
+                double alpha) {
   SEQ_IN(p);
   TORCH_CHECK(p.dim() == 2 && col >= 0 && N >= 1 &&
-                  col + 2 * N <= p.size(1) && act >= 0 && act <= 2,
+                  col + 2 * N <= p.size(1) && act >= 0 && act <= 4,
               "p must hold 2N columns from col");
   auto out = torch::empty({p.size(0), N}, p.options());
   tl_act_gate((const char*)p.data_ptr() + col * p.element_size(), p.size(1),
               p.size(1) % 8 == 0 && col % 8 == 0, out.data_ptr(), p.size(0),
-              (int)N, (int)act, act_is_f32(p), seq_stream());
+              (int)N, (int)act, (float)lim, (float)alpha, act_is_f32(p),
+              seq_stream());
   return out;
 }
 
-// per head: x_h / rms(x_h) * w [* silu(gate columns)], x fp32 [T, H*V]
+// per head: x_h / rms(x_h) * w [* silu | sigmoid of the gate columns], x fp32
+// [T, H*V]
 Tensor head_rms_gate(Tensor x, Tensor w, int64_t H, double eps,
                      c10::optional<Tensor> gate, int64_t gate_col,
-                     bool out_f32) {
+                     bool sig, bool out_f32) {
   SEQ_F32(x);
   SEQ_F32(w);
   const int64_t V = w.numel();
@@ -226,8 +242,8 @@ Tensor head_rms_gate(Tensor x, Tensor w, int64_t H, double eps,
       x.options().dtype(out_f32 ? torch::kFloat : torch::kBFloat16));
   tl_head_rms_gate(x.data_ptr(), w.data_ptr(), gp, ldg,
                    ldg % 4 == 0 && gate_col % 4 == 0, out.data_ptr(),
-                   x.size(0), (int)H, (int)V, (float)eps, out_f32 ? 1 : 0,
-                   seq_stream());
+                   x.size(0), (int)H, (int)V, (float)eps, sig ? 1 : 0,
+                   out_f32 ? 1 : 0, seq_stream());
   return out;
 }
 

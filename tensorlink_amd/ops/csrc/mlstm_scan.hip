@@ -46,7 +46,8 @@ template <typename T, int DMAX, int TB, int DG>
 __global__ __launch_bounds__(1024) void mlstm_seq_kernel(
     const T* __restrict__ proj, int ld, int q_off, int k_off, int v_off,
     int g_off,
-    const float* __restrict__ gates,   // [Ttot, 2H] raw (input | forget)
+    const float* __restrict__ gates,   // [Ttot, ldg]: raw input [H] | forget
+    int ldg,                           // [H] in the first 2H columns
     const float* __restrict__ norm_w,  // [H*V]
     float* __restrict__ S_pool,        // [slots, H, D, V]
     float* __restrict__ n_pool,        // [slots, H, D]
@@ -120,8 +121,8 @@ __global__ __launch_bounds__(1024) void mlstm_seq_kernel(
     }
     if (threadIdx.x < cnt) {
       const int tt = threadIdx.x;
-      const float gi = gates[(int64_t)(tb0 + tt) * 2 * H + h];
-      const float gf = gates[(int64_t)(tb0 + tt) * 2 * H + H + h];
+      const float gi = gates[(int64_t)(tb0 + tt) * ldg + h];
+      const float gf = gates[(int64_t)(tb0 + tt) * ldg + H + h];
       lli[tt] = cap * tanhf(gi / cap);
       llf[tt] = log_sigmoid(cap * tanhf(gf / cap));
     }
@@ -308,8 +309,8 @@ extern "C" {
 
 // returns 0 on success, 1 if the shape is outside what the kernel serves
 int tl_mlstm_seq(const void* proj, int ld, int q_off, int k_off, int v_off,
-                 int g_off, const void* gates, const void* norm_w, void* S,
-                 void* n, void* m, const void* cu, const void* slots,
+                 int g_off, const void* gates, int ldg, const void* norm_w,
+                 void* S, void* n, void* m, const void* cu, const void* slots,
                  const void* pos0, void* out, int B, int H, int D, int V,
                  float cap, float qscale, float eps, void* F, int summary,
                  int is_f32, hipStream_t stream) {
@@ -324,7 +325,7 @@ int tl_mlstm_seq(const void* proj, int ld, int q_off, int k_off, int v_off,
                                          (DGG > 1 ? TBB * DGG * nc : 0));    \
     hipLaunchKernelGGL((mlstm_seq_kernel<TT, DM, TBB, DGG>), grid,           \
                        dim3(nc * DGG), smem, stream, (const TT*)proj, ld,    \
-                       q_off, k_off, v_off, g_off, (const float*)gates,      \
+                       q_off, k_off, v_off, g_off, (const float*)gates, ldg, \
                        (const float*)norm_w, (float*)S, (float*)n,           \
                        (float*)m, (const int*)cu, (const int*)slots,         \
                        (const int*)pos0, (TT*)out, H, D, V, cap, qscale,     \

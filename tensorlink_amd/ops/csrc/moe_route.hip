@@ -1,6 +1,7 @@
 // Routing of a mixture of experts (gfx950): fp32 router logits, selection of
-// the largest ones with a softmax over the chosen, expert-sorted (token,
-// choice) pairs, a grouped product for shapes and dtypes that the MFMA
+// the largest ones with a softmax over the chosen (or scores from a softmax
+// over all experts, chosen with a correction), expert-sorted (token, choice)
+// pairs, a grouped product for shapes and dtypes that the MFMA
 // kernel (moe_gemm.hip) does not take, and the weighted combine.
 //
 // The position of a pair inside its expert's segment is handed out by LDS
@@ -25,19 +26,20 @@ template <typename T> DEVINLINE void stf(T* p, float v);
 template <> DEVINLINE void stf<float>(float* p, float v) { *p = v; }
 template <> DEVINLINE void stf<bf16>(bf16* p, float v) { *p = f2bf(v); }
 
-// one wave: the `top` largest of z[0..E), the lower index first among equals
-DEVINLINE void select_top(const float* z, int E, int top, float* wt,
-                          int* idx) {
+// one wave: the `top` largest of val(0..E-1), the lower index first among
+// equals; lane j receives the j-th chosen value and its index
+template <typename F>
+DEVINLINE void pick_top(F val, int E, int top, float& mine, int& mine_e) {
   const int lane = threadIdx.x & (WAVE_SIZE - 1);
   unsigned taken = 0;
-  float mine = 0.f;                  // lane j: the j-th chosen logit
-  int mine_e = 0;
+  mine = 0.f;
+  mine_e = 0;
   for (int j = 0; j < top; ++j) {
     float best = -INFINITY;
     int be = 0x7fffffff;
     for (int e = lane, k = 0; e < E; e += WAVE_SIZE, ++k) {
       if (taken & (1u << k)) continue;
-      float v = z[e];
+      float v = val(e);
       if (!(v > -INFINITY)) v = -INFINITY;       // NaN counts as smallest
       if (v > best || (v == best && e < be)) {
         best = v;
@@ -59,6 +61,15 @@ DEVINLINE void select_top(const float* z, int E, int top, float* wt,
       mine_e = be;
     }
   }
+}
+
+// the `top` largest logits, weighted by the softmax over the chosen ones
+DEVINLINE void select_top(const float* z, int E, int top, float* wt,
+                          int* idx) {
+  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+  float mine;
+  int mine_e;
+  pick_top([&](int e) { return z[e]; }, E, top, mine, mine_e);
   const float m = __shfl(mine, 0, WAVE_SIZE);    // the largest comes first
   const float ex = lane < top ? expf(mine - m) : 0.f;
   const float tot = wave_reduce_sum(ex);
@@ -137,6 +148,33 @@ __global__ __launch_bounds__(BLOCK) void route_logits_vec_kernel(
   __syncthreads();
   if (threadIdx.x < WAVE_SIZE)
     select_top(z, E, top, wt + t * top, idx + t * top);
+}
+
+// one wave per token, logits given (rows of stride ldz): scores s = softmax
+// over all experts, chosen by s + corr, weighted by s
+__global__ __launch_bounds__(BLOCK) void route_scores_kernel(
+    const float* __restrict__ z, int64_t ldz, const float* __restrict__ corr,
+    float* __restrict__ wt, int* __restrict__ idx, int64_t T, int E,
+    int top) {
+  const int64_t t = (int64_t)blockIdx.x * NWAVE + threadIdx.x / WAVE_SIZE;
+  if (t >= T) return;
+  const int lane = threadIdx.x & (WAVE_SIZE - 1);
+  const float* zr = z + t * ldz;
+  float m = -INFINITY;
+  for (int e = lane; e < E; e += WAVE_SIZE) m = fmaxf(m, zr[e]);
+  m = wave_reduce_max(m);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += WAVE_SIZE) sum += expf(zr[e] - m);
+  const float inv = 1.f / wave_reduce_sum(sum);
+  float mine;
+  int me;
+  pick_top([&](int e) { return expf(zr[e] - m) * inv + (corr ? corr[e] : 0.f); },
+           E, top, mine, me);
+  if (lane < top) {
+    me = min(me, E - 1);
+    wt[t * top + lane] = expf(zr[me] - m) * inv;
+    idx[t * top + lane] = me;
+  }
 }
 
 // one wave per token, logits given
@@ -284,14 +322,18 @@ __global__ __launch_bounds__(BLOCK) void grouped_any_kernel(
 }
 
 // --------------------------------------------------------------- combine
-// out[t] = sum_j wt[t][j] y[rank[t][j]] (+ sigmoid(sg[t]) * shared[t])
+// out[t] = sum_j wt[t][j] y[rank[t][j]] (+ sigmoid(sg[t]) * shared[t]). With
+// `ident` [T, W] the pairs at sorted positions >= *n_real belong to identity
+// experts, whose output is the token's own row of it.
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void combine_kernel(
     const T* __restrict__ y, const int* __restrict__ rank,
     const float* __restrict__ wt, const T* __restrict__ shared,
-    const T* __restrict__ sg, int ldg, int sg_col, T* __restrict__ out,
-    int W, int top) {
+    const T* __restrict__ sg, int ldg, int sg_col,
+    const T* __restrict__ ident, const int* __restrict__ n_real,
+    T* __restrict__ out, int W, int top) {
   const int64_t t = blockIdx.x;
+  const int real = ident ? *n_real : 0x7fffffff;
   float f = 0.f;
   if (shared) {
     f = 1.f;
@@ -300,8 +342,11 @@ __global__ __launch_bounds__(BLOCK) void combine_kernel(
   for (int c = blockIdx.y * BLOCK + threadIdx.x; c < W;
        c += gridDim.y * BLOCK) {
     float a = 0.f;
-    for (int j = 0; j < top; ++j)
-      a += wt[t * top + j] * ldf<T>(y + (int64_t)rank[t * top + j] * W + c);
+    for (int j = 0; j < top; ++j) {
+      const int r = rank[t * top + j];
+      const T* src = r < real ? y + (int64_t)r * W : ident + t * W;
+      a += wt[t * top + j] * ldf<T>(src + c);
+    }
     if (shared) a += f * ldf<T>(shared + t * W + c);
     stf<T>(out + t * W + c, a);
   }
@@ -311,9 +356,11 @@ __global__ __launch_bounds__(BLOCK) void combine_kernel(
 __global__ __launch_bounds__(BLOCK) void combine_vec8_kernel(
     const bf16* __restrict__ y, const int* __restrict__ rank,
     const float* __restrict__ wt, const bf16* __restrict__ shared,
-    const bf16* __restrict__ sg, int ldg, int sg_col, bf16* __restrict__ out,
-    int64_t n8, int W, int top) {
+    const bf16* __restrict__ sg, int ldg, int sg_col,
+    const bf16* __restrict__ ident, const int* __restrict__ n_real,
+    bf16* __restrict__ out, int64_t n8, int W, int top) {
   const int W8 = W / 8;
+  const int real = ident ? *n_real : 0x7fffffff;
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n8;
        i += (int64_t)gridDim.x * BLOCK) {
     const int64_t t = i / W8;
@@ -321,8 +368,9 @@ __global__ __launch_bounds__(BLOCK) void combine_vec8_kernel(
     float a[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     for (int j = 0; j < top; ++j) {
       const float w = wt[t * top + j];
-      const bf16x8 v = *reinterpret_cast<const bf16x8*>(
-          y + (int64_t)rank[t * top + j] * W + c);
+      const int r = rank[t * top + j];
+      const bf16* src = r < real ? y + (int64_t)r * W : ident + t * W;
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(src + c);
 #pragma unroll
       for (int e = 0; e < 8; ++e) a[e] += w * bf2f(v.v[e]);
     }
@@ -384,6 +432,17 @@ void tl_moe_route(const void* h, const void* w, const void* z, void* wt,
                        (int*)idx, W, E, top);
 }
 
+// z: first logit of row 0, rows of stride ldz; corr [E] or null
+void tl_moe_route_scores(const void* z, int64_t ldz, const void* corr,
+                         void* wt, void* idx, int64_t T, int E, int top,
+                         hipStream_t stream) {
+  if (T <= 0) return;
+  hipLaunchKernelGGL(route_scores_kernel,
+                     dim3((unsigned)((T + NWAVE - 1) / NWAVE)), dim3(BLOCK), 0,
+                     stream, (const float*)z, ldz, (const float*)corr,
+                     (float*)wt, (int*)idx, T, E, top);
+}
+
 // blocks whose counts the caller's scratch [blocks][E] must hold (0: none)
 int tl_moe_sort_blocks(int P) { return P <= TILE ? 0 : (P + TILE - 1) / TILE; }
 
@@ -425,7 +484,8 @@ void tl_grouped_any(const void* x, const void* tok_idx, const void* seg,
 
 void tl_moe_combine(const void* y, const void* rank, const void* wt,
                     const void* shared, const void* sg, int ldg, int sg_col,
-                    void* out, int64_t T, int W, int top, int is_f32,
+                    const void* ident, const void* n_real, void* out,
+                    int64_t T, int W, int top, int is_f32,
                     hipStream_t stream) {
   if (T <= 0) return;
   if (!is_f32 && W % 8 == 0) {
@@ -435,7 +495,8 @@ void tl_moe_combine(const void* y, const void* rank, const void* wt,
                        dim3((unsigned)(nb > 8192 ? 8192 : nb)), dim3(BLOCK), 0,
                        stream, (const bf16*)y, (const int*)rank,
                        (const float*)wt, (const bf16*)shared, (const bf16*)sg,
-                       ldg, sg_col, (bf16*)out, n8, W, top);
+                       ldg, sg_col, (const bf16*)ident, (const int*)n_real,
+                       (bf16*)out, n8, W, top);
     return;
   }
   const int cb = (W + BLOCK - 1) / BLOCK;
@@ -444,12 +505,14 @@ void tl_moe_combine(const void* y, const void* rank, const void* wt,
     hipLaunchKernelGGL(combine_kernel<float>, grid, block, 0, stream,
                        (const float*)y, (const int*)rank, (const float*)wt,
                        (const float*)shared, (const float*)sg, ldg, sg_col,
-                       (float*)out, W, top);
+                       (const float*)ident, (const int*)n_real, (float*)out,
+                       W, top);
   else
     hipLaunchKernelGGL(combine_kernel<bf16>, grid, block, 0, stream,
                        (const bf16*)y, (const int*)rank, (const float*)wt,
                        (const bf16*)shared, (const bf16*)sg, ldg, sg_col,
-                       (bf16*)out, W, top);
+                       (const bf16*)ident, (const int*)n_real, (bf16*)out, W,
+                       top);
 }
 
 }  // extern "C"

@@ -17,9 +17,11 @@
 // of the sublayer's own projection in the same pass. Rows of a multiple of 4
 // columns are held in registers between the statistic and the scaling.
 // tl_act_gate is the gated feed-forward's activation on a fused [gate | up]
-// projection: act(gate) * up, act = gelu (erf / tanh form) or silu.
-// tl_head_rms_gate is the read-out norm of a linear-attention mixer whose
-// heads are normed on their own: x_h / rms(x_h) * w [* silu(gate)].
+// projection: act(gate) * up, act = gelu (erf / tanh form), silu or relu, or
+// the clamped swish. A residual sum may have up to three terms, each with a
+// factor (sublayers side by side). tl_head_rms_gate is the read-out norm of a
+// linear-attention mixer whose heads are normed on their own:
+// x_h / rms(x_h) * w [* silu(gate) | sigmoid(gate)].
 
 #include "common.hpp"
 
@@ -67,6 +69,14 @@ __global__ __launch_bounds__(BLOCK) void postnorm_add_kernel(
   }
 }
 
+// further terms of a residual sum beside the first, and every term's factor
+template <typename T>
+struct AddMore {
+  const T* y1;
+  const T* y2;
+  float s0, s1, s2;
+};
+
 // y[c] [* sigmoid(gate[c])]
 template <typename T>
 DEVINLINE float gated(const T* y, const T* gate, int64_t c) {
@@ -74,12 +84,13 @@ DEVINLINE float gated(const T* y, const T* gate, int64_t c) {
   return gate ? v / (1.f + expf(-ldf<T>(gate, c))) : v;
 }
 
-// X += y (if given); h = X / rms(X) * w in the serving dtype (no w: no h)
+// X += sum of the given terms; h = X / rms(X) * w in the serving dtype (no w:
+// no h)
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void add_rms_kernel(
     float* __restrict__ X, const T* __restrict__ y,
     const float* __restrict__ w, T* __restrict__ h, int W, float eps,
-    float x_scale, const T* __restrict__ gate, int ldg) {
+    float x_scale, const T* __restrict__ gate, int ldg, AddMore<T> more) {
   __shared__ float red[NW];
   const int64_t row = blockIdx.x;
   float* xr = X + row * W;
@@ -88,7 +99,9 @@ __global__ __launch_bounds__(BLOCK) void add_rms_kernel(
   float ss = 0.f;
   for (int c = threadIdx.x; c < W; c += BLOCK) {
     float v = xr[c] * x_scale;
-    if (y) v += gated<T>(yr, gr, c);
+    if (y) v += more.s0 * gated<T>(yr, gr, c);
+    if (more.y1) v += more.s1 * ldf<T>(more.y1, row * W + c);
+    if (more.y2) v += more.s2 * ldf<T>(more.y2, row * W + c);
     if (y || x_scale != 1.f) xr[c] = v;
     ss += v * v;
   }
@@ -131,7 +144,7 @@ template <typename T, int NV>
 __global__ __launch_bounds__(BLOCK) void add_rms_vec_kernel(
     float* __restrict__ X, const T* __restrict__ y,
     const float* __restrict__ w, T* __restrict__ h, int W, float eps,
-    float x_scale, const T* __restrict__ gate, int ldg) {
+    float x_scale, const T* __restrict__ gate, int ldg, AddMore<T> more) {
   __shared__ float red[NW];
   const int64_t row = blockIdx.x;
   float* xr = X + row * W;
@@ -156,7 +169,19 @@ __global__ __launch_bounds__(BLOCK) void add_rms_vec_kernel(
           for (int e = 0; e < 4; ++e) u[e] = u[e] / (1.f + expf(-g[e]));
         }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) v[k][e] += u[e];
+        for (int e = 0; e < 4; ++e) v[k][e] += more.s0 * u[e];
+      }
+      if (more.y1) {
+        float u[4];
+        ld4(more.y1 + row * W + c, u);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[k][e] += more.s1 * u[e];
+      }
+      if (more.y2) {
+        float u[4];
+        ld4(more.y2 + row * W + c, u);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[k][e] += more.s2 * u[e];
       }
       if (y || x_scale != 1.f) st4(xr + c, v[k]);
 #pragma unroll
@@ -182,11 +207,11 @@ __global__ __launch_bounds__(BLOCK) void add_rms_vec_kernel(
 template <typename T>
 void launch_add_rms(float* X, const T* y, const float* w, T* h, int64_t rows,
                     int W, float eps, float x_scale, const T* gate, int ldg,
-                    bool vec, hipStream_t stream) {
+                    AddMore<T> more, bool vec, hipStream_t stream) {
   dim3 grid((unsigned)rows), block(BLOCK);
 #define TL_AR(NV)                                                           \
   hipLaunchKernelGGL((add_rms_vec_kernel<T, NV>), grid, block, 0, stream, X, \
-                     y, w, h, W, eps, x_scale, gate, ldg)
+                     y, w, h, W, eps, x_scale, gate, ldg, more)
   const int nv = (W / 4 + BLOCK - 1) / BLOCK;
   if (vec && nv <= 1) TL_AR(1);
   else if (vec && nv <= 2) TL_AR(2);
@@ -194,34 +219,43 @@ void launch_add_rms(float* X, const T* y, const float* w, T* h, int64_t rows,
   else if (vec && nv <= 8) TL_AR(8);
   else
     hipLaunchKernelGGL(add_rms_kernel<T>, grid, block, 0, stream, X, y, w, h,
-                       W, eps, x_scale, gate, ldg);
+                       W, eps, x_scale, gate, ldg, more);
 #undef TL_AR
 }
 
-// act(z): 0 erf GELU, 1 tanh-form GELU, 2 silu
-DEVINLINE float act_f(float z, int act) {
-  if (act == 2) return z / (1.f + expf(-z));
-  return gelu_f(z, act);
+// a gated feed-forward's activation of (gate g, up u): 0 erf GELU, 1
+// tanh-form GELU, 2 silu, 3 relu, times u; 4 the clamped swish, with g <=
+// lim and |u| <= lim, g sigmoid(alpha g) (u + 1)
+DEVINLINE float pair_act(float g, float u, int act, float lim, float alpha) {
+  if (act == 4) {
+    g = fminf(g, lim);
+    u = fminf(fmaxf(u, -lim), lim);
+    return g / (1.f + expf(-alpha * g)) * (u + 1.f);
+  }
+  if (act == 3) return fmaxf(g, 0.f) * u;
+  if (act == 2) return g / (1.f + expf(-g)) * u;
+  return gelu_f(g, act) * u;
 }
 
-// out[r][c] = act(p[r][c]) * p[r][N + c] on rows of stride ld
+// out[r][c] = pair_act(p[r][c], p[r][N + c]) on rows of stride ld
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void act_gate_kernel(
     const T* __restrict__ p, int64_t ld, T* __restrict__ out, int64_t n,
-    int N, int act) {
+    int N, int act, float lim, float alpha) {
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n;
        i += (int64_t)gridDim.x * BLOCK) {
     const int64_t r = i / N;
     const int c = (int)(i - r * N);
     const T* row = p + r * ld;
-    stf<T>(out, i, act_f(ldf<T>(row, c), act) * ldf<T>(row, N + c));
+    stf<T>(out, i,
+           pair_act(ldf<T>(row, c), ldf<T>(row, N + c), act, lim, alpha));
   }
 }
 
 // bf16, N, the stride and the first column multiples of 8: 16-byte accesses
 __global__ __launch_bounds__(BLOCK) void act_gate_vec8_kernel(
     const bf16x8* __restrict__ p, int64_t ld8, bf16x8* __restrict__ out,
-    int64_t n8, int N8, int act) {
+    int64_t n8, int N8, int act, float lim, float alpha) {
   for (int64_t i = (int64_t)blockIdx.x * BLOCK + threadIdx.x; i < n8;
        i += (int64_t)gridDim.x * BLOCK) {
     const int64_t r = i / N8;
@@ -230,17 +264,18 @@ __global__ __launch_bounds__(BLOCK) void act_gate_vec8_kernel(
     bf16x8 o;
 #pragma unroll
     for (int e = 0; e < 8; ++e)
-      o.v[e] = f2bf(act_f(bf2f(a.v[e]), act) * bf2f(b.v[e]));
+      o.v[e] = f2bf(pair_act(bf2f(a.v[e]), bf2f(b.v[e]), act, lim, alpha));
     out[i] = o;
   }
 }
 
-// one wave per (row, head): out = x_h / rms(x_h) * w [* silu(gate)]
+// one wave per (row, head): out = x_h / rms(x_h) * w [* silu(gate), or
+// sigmoid(gate) with sig]
 template <typename T>
 __global__ __launch_bounds__(BLOCK) void head_rms_gate_kernel(
     const float* __restrict__ x, const float* __restrict__ w,
     const T* __restrict__ gate, int ldg, T* __restrict__ out, int64_t units,
-    int H, int V, float eps) {
+    int H, int V, float eps, int sig) {
   const int64_t u = (int64_t)blockIdx.x * NW + threadIdx.x / WAVE_SIZE;
   if (u >= units) return;
   const int lane = threadIdx.x & (WAVE_SIZE - 1);
@@ -254,7 +289,7 @@ __global__ __launch_bounds__(BLOCK) void head_rms_gate_kernel(
     float v = xr[c] * rn * w[c];
     if (gate) {
       const float z = ldf<T>(gr, c);
-      v *= z / (1.f + expf(-z));
+      v *= (sig ? 1.f : z) / (1.f + expf(-z));
     }
     stf<T>(out, u * V + c, v);
   }
@@ -266,7 +301,7 @@ template <typename T>
 __global__ __launch_bounds__(BLOCK) void head_rms_gate_vec_kernel(
     const float* __restrict__ x, const float* __restrict__ w,
     const T* __restrict__ gate, int ldg, T* __restrict__ out, int64_t units,
-    int H, int V, float eps, int LG) {
+    int H, int V, float eps, int LG, int sig) {
   const int64_t u = ((int64_t)blockIdx.x * BLOCK + threadIdx.x) / LG;
   const bool on = u < units;      // a wave's lanes shuffle together
   const int c0 = (threadIdx.x & (LG - 1)) * 4;
@@ -294,7 +329,8 @@ __global__ __launch_bounds__(BLOCK) void head_rms_gate_vec_kernel(
       float z[4];
       ld4(gr + c, z);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] *= z[e] / (1.f + expf(-z[e]));
+      for (int e = 0; e < 4; ++e)
+        v[e] *= (sig ? 1.f : z[e]) / (1.f + expf(-z[e]));
     }
     st4(out + u * V + c, v);
   }
@@ -302,12 +338,12 @@ __global__ __launch_bounds__(BLOCK) void head_rms_gate_vec_kernel(
 
 template <typename T>
 void launch_head_rms(const float* x, const float* w, const T* gate, int ldg,
-                     T* out, int64_t units, int H, int V, float eps, bool vec,
-                     hipStream_t stream) {
+                     T* out, int64_t units, int H, int V, float eps, int sig,
+                     bool vec, hipStream_t stream) {
   if (!vec) {
     hipLaunchKernelGGL(head_rms_gate_kernel<T>,
                        dim3((unsigned)((units + NW - 1) / NW)), dim3(BLOCK), 0,
-                       stream, x, w, gate, ldg, out, units, H, V, eps);
+                       stream, x, w, gate, ldg, out, units, H, V, eps, sig);
     return;
   }
   int LG = 1;
@@ -315,7 +351,7 @@ void launch_head_rms(const float* x, const float* w, const T* gate, int ldg,
   hipLaunchKernelGGL(head_rms_gate_vec_kernel<T>,
                      dim3((unsigned)((units * LG + BLOCK - 1) / BLOCK)),
                      dim3(BLOCK), 0, stream, x, w, gate, ldg, out, units, H, V,
-                     eps, LG);
+                     eps, LG, sig);
 }
 
 // out = x / rms(x) * g [* sigmoid(gate)], x fp32 [rows, N]
@@ -407,56 +443,64 @@ void tl_postnorm_add(void* X, const void* y, const void* w, void* h,
                        W, eps, one_plus);
 }
 
-// gate: first gate column of row 0 (rows of stride ldg), or null
+// gate: first gate column of row 0 (rows of stride ldg), or null; y, y1, y2
+// enter the sum times s0, s1, s2
 void tl_add_rms(void* X, const void* y, const void* w, void* h, int64_t rows,
                 int W, float eps, float x_scale, const void* gate, int ldg,
-                int gate_aligned, int is_f32, hipStream_t stream) {
+                int gate_aligned, float s0, const void* y1, float s1,
+                const void* y2, float s2, int is_f32, hipStream_t stream) {
   if (rows <= 0) return;
   const bool vec = W % 4 == 0 && (!gate || gate_aligned);
   if (is_f32)
     launch_add_rms<float>((float*)X, (const float*)y, (const float*)w,
                           (float*)h, rows, W, eps, x_scale,
-                          (const float*)gate, ldg, vec, stream);
+                          (const float*)gate, ldg,
+                          AddMore<float>{(const float*)y1, (const float*)y2,
+                                         s0, s1, s2},
+                          vec, stream);
   else
     launch_add_rms<bf16>((float*)X, (const bf16*)y, (const float*)w, (bf16*)h,
-                         rows, W, eps, x_scale, (const bf16*)gate, ldg, vec,
-                         stream);
+                         rows, W, eps, x_scale, (const bf16*)gate, ldg,
+                         AddMore<bf16>{(const bf16*)y1, (const bf16*)y2, s0,
+                                       s1, s2},
+                         vec, stream);
 }
 
 // p: first gate column of row 0, rows of stride ld
 void tl_act_gate(const void* p, int64_t ld, int aligned, void* out,
-                 int64_t rows, int N, int act, int is_f32,
-                 hipStream_t stream) {
+                 int64_t rows, int N, int act, float lim, float alpha,
+                 int is_f32, hipStream_t stream) {
   const int64_t n = rows * N;
   if (n <= 0) return;
   if (!is_f32 && aligned && N % 8 == 0) {
     hipLaunchKernelGGL(act_gate_vec8_kernel, dim3(ew_grid(n / 8)),
                        dim3(BLOCK), 0, stream, (const bf16x8*)p, ld / 8,
-                       (bf16x8*)out, n / 8, N / 8, act);
+                       (bf16x8*)out, n / 8, N / 8, act, lim, alpha);
     return;
   }
   dim3 grid(ew_grid(n)), block(BLOCK);
   if (is_f32)
     hipLaunchKernelGGL(act_gate_kernel<float>, grid, block, 0, stream,
-                       (const float*)p, ld, (float*)out, n, N, act);
+                       (const float*)p, ld, (float*)out, n, N, act, lim, alpha);
   else
     hipLaunchKernelGGL(act_gate_kernel<bf16>, grid, block, 0, stream,
-                       (const bf16*)p, ld, (bf16*)out, n, N, act);
+                       (const bf16*)p, ld, (bf16*)out, n, N, act, lim, alpha);
 }
 
 void tl_head_rms_gate(const void* x, const void* w, const void* gate, int ldg,
                       int gate_aligned, void* out, int64_t rows, int H, int V,
-                      float eps, int is_f32, hipStream_t stream) {
+                      float eps, int sig, int is_f32, hipStream_t stream) {
   const int64_t units = rows * H;
   if (units <= 0) return;
   const bool vec = V % 4 == 0 && (!gate || gate_aligned);
   if (is_f32)
     launch_head_rms<float>((const float*)x, (const float*)w,
                            (const float*)gate, ldg, (float*)out, units, H, V,
-                           eps, vec, stream);
+                           eps, sig, vec, stream);
   else
     launch_head_rms<bf16>((const float*)x, (const float*)w, (const bf16*)gate,
-                          ldg, (bf16*)out, units, H, V, eps, vec, stream);
+                          ldg, (bf16*)out, units, H, V, eps, sig, vec,
+                          stream);
 }
 
 void tl_rms_scale(const void* x, const void* w, const void* gate, int ldg,

@@ -187,8 +187,9 @@ def mlstm_scan(proj: torch.Tensor, offs, gates: torch.Tensor,
                cap: float, eps: float) -> torch.Tensor:
     """Stabilised matrix-memory recurrence for every sequence of the step.
 
-    proj [T, L] holds q | k | v | g at column offsets ``offs``; gates
-    [T, 2H] fp32 are the raw input | forget pre-activations. State pools
+    proj [T, L] holds q | k | v | g at column offsets ``offs``; the first
+    2H columns of gates (fp32) are the raw input | forget pre-activations.
+    State pools
     S [slots, H, D, V], n [slots, H, D], m [slots, H] (fp32) are read at
     ``meta.slots`` (zero for a sequence with no cached tokens) and written
     back. Returns [T, H*V]: per-head unit-RMS of the read-out, times
@@ -233,7 +234,7 @@ def mlstm_scan(proj: torch.Tensor, offs, gates: torch.Tensor,
     v = pf[:, v_off:v_off + H * V].view(T, H, V)
     g = pf[:, g_off:g_off + H * V]
     li = soft_cap(gates[:, :H], cap)
-    lf = torch.nn.functional.logsigmoid(soft_cap(gates[:, H:], cap))
+    lf = torch.nn.functional.logsigmoid(soft_cap(gates[:, H:2 * H], cap))
     o = torch.empty(T, H, V)
     for b in range(meta.B):
         slot = meta.slots_h[b]
@@ -390,23 +391,27 @@ def postnorm_add(X: torch.Tensor, y: torch.Tensor, w: torch.Tensor,
 
 def rms_scale(x: torch.Tensor, w: torch.Tensor, eps: float, one_plus: bool,
               gate: Optional[torch.Tensor] = None, gate_col: int = 0,
-              out_dtype=torch.float32, heads: int = 0) -> torch.Tensor:
+              out_dtype=torch.float32, heads: int = 0,
+              gate_act: str = "silu") -> torch.Tensor:
     """x / rms(x) * (1 + w | w) over the last axis of x [T, N] (fp32),
     optionally times sigmoid(gate[:, gate_col:gate_col + N]). With ``heads``
     > 0 every one of that many equal parts of a row has its own statistic,
     the weight [N / heads] is shared by them, and the gate goes through
-    silu instead of the sigmoid."""
+    ``gate_act``, "silu" or "sigmoid"."""
     assert x.dtype == torch.float32 and w.dtype == torch.float32
     if heads:
         assert not one_plus and x.shape[1] == heads * w.numel()
+        assert gate_act in ("silu", "sigmoid")
         if x.is_cuda:
             return _ext().head_rms_gate(
                 x.contiguous(), w, int(heads), float(eps), gate,
-                int(gate_col), out_dtype == torch.float32)
+                int(gate_col), gate_act == "sigmoid",
+                out_dtype == torch.float32)
         y = (_rms(x.view(x.shape[0], heads, -1), eps) * w).reshape(x.shape)
         if gate is not None:
-            y = y * torch.nn.functional.silu(
-                gate[:, gate_col:gate_col + x.shape[1]].float())
+            z = gate[:, gate_col:gate_col + x.shape[1]].float()
+            y = y * (torch.sigmoid(z) if gate_act == "sigmoid"
+                     else torch.nn.functional.silu(z))
         return y.to(out_dtype)
     if x.is_cuda:
         return _ext().rms_scale(x.contiguous(), w, float(eps),
@@ -451,7 +456,8 @@ def soft_cap_(z: torch.Tensor, cap: float, scale: float = 1.0) -> torch.Tensor:
 def add_rms(X: torch.Tensor, y: Optional[torch.Tensor],
             w: Optional[torch.Tensor], eps: float, out_dtype=torch.float32,
             x_scale: float = 1.0, gate: Optional[torch.Tensor] = None,
-            gate_col: int = 0) -> torch.Tensor:
+            gate_col: int = 0, y_scale: float = 1.0,
+            more: Sequence[tuple] = ()) -> torch.Tensor:
     """Pre-norm residual step, in place on the fp32 residual X [T, W]:
     X <- X * x_scale + y (``y`` = the previous sublayer's output, or None),
     then returns the next sublayer's input X / rms(X) * w in ``out_dtype``;
@@ -459,15 +465,19 @@ def add_rms(X: torch.Tensor, y: Optional[torch.Tensor],
     returned. With ``gate`` [T, L] y is first multiplied, element by
     element, by sigmoid(gate[:, gate_col:gate_col + W]) (a gated residual;
     the pre-activations are columns of the sublayer's own projection).
+    ``y_scale`` multiplies y; ``more`` holds up to two further (tensor,
+    factor) terms of the sum (sublayers that read the same input).
     Sum, sigmoid, statistic and scaling are fp32."""
     assert X.dtype == torch.float32
+    assert len(more) <= 2 and (y is not None or not more)
     assert w is None or w.dtype == torch.float32
     assert gate is None or y is not None
     if X.is_cuda:
+        (y1, s1), (y2, s2) = tuple(more) + ((None, 0.0),) * (2 - len(more))
         return _ext().add_rms(
             X, None if y is None else y.contiguous(), w, float(eps),
-            float(x_scale), gate, int(gate_col),
-            out_dtype == torch.float32)
+            float(x_scale), gate, int(gate_col), float(y_scale), y1,
+            float(s1), y2, float(s2), out_dtype == torch.float32)
     if x_scale != 1.0:
         X *= x_scale
     if y is not None:
@@ -475,28 +485,51 @@ def add_rms(X: torch.Tensor, y: Optional[torch.Tensor],
         if gate is not None:
             u = u * torch.sigmoid(
                 gate[:, gate_col:gate_col + X.shape[1]].float())
-        X += u
+        X += u if y_scale == 1.0 else y_scale * u
+    for m, f in more:
+        X += float(f) * m.float()
     return X if w is None else (_rms(X, eps) * w).to(out_dtype)
 
 
-GATE_ACTS = {"gelu": 0, "gelu_tanh": 1, "silu": 2}
+GATE_ACTS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3,
+             "clamped_swish": 4}
 
 
-def act_gate(p: torch.Tensor, act: str, N: int = 0,
+def _act_code(act):
+    """(code, limit, alpha) of an activation name, or of the tuple
+    ("clamped_swish", limit, alpha)."""
+    if isinstance(act, str):
+        assert act != "clamped_swish", "needs its limit and alpha"
+        return GATE_ACTS[act], 0.0, 0.0
+    name, limit, alpha = act
+    assert name == "clamped_swish"
+    return GATE_ACTS[name], float(limit), float(alpha)
+
+
+def act_gate(p: torch.Tensor, act, N: int = 0,
              col: int = 0) -> torch.Tensor:
     """act(p[:, col:col + N]) * p[:, col + N:col + 2N] for a fused
     projection p [T, L] that holds [gate | up] from column ``col`` (N = 0:
-    the whole of p); ``act`` is "gelu" (erf), "gelu_tanh" or "silu".
+    the whole of p); ``act`` is "gelu" (erf), "gelu_tanh", "silu", "relu",
+    or ("clamped_swish", limit, alpha): with g = min(gate, limit) and
+    u = clamp(up, -limit, limit), g sigmoid(alpha g) (u + 1).
     Evaluated in fp32, result [T, N] in p's dtype."""
     N = N or p.shape[1] // 2
+    code, limit, alpha = _act_code(act)
     if p.is_cuda:
-        return _ext().act_gate(p.contiguous(), int(col), int(N),
-                               GATE_ACTS[act])
+        return _ext().act_gate(p.contiguous(), int(col), int(N), code, limit,
+                               alpha)
     g = p[:, col:col + N].float()
+    u = p[:, col + N:col + 2 * N].float()
     F = torch.nn.functional
-    y = F.silu(g) if act == "silu" else F.gelu(
-        g, approximate="tanh" if act == "gelu_tanh" else "none")
-    return (y * p[:, col + N:col + 2 * N].float()).to(p.dtype)
+    if code == 4:
+        g = g.clamp(max=limit)
+        return (g * torch.sigmoid(alpha * g)
+                * (u.clamp(-limit, limit) + 1.0)).to(p.dtype)
+    y = (F.silu(g) if act == "silu" else F.relu(g) if act == "relu"
+         else F.gelu(g, approximate="tanh" if act == "gelu_tanh"
+                     else "none"))
+    return (y * u).to(p.dtype)
 
 
 def gelu_gate(p: torch.Tensor, tanh_form: bool = True) -> torch.Tensor:
@@ -1189,23 +1222,44 @@ def topk_softmax_router(h: torch.Tensor, w: torch.Tensor, top: int):
     return torch.softmax(z.gather(1, idx), -1), idx.to(torch.int32)
 
 
+def score_router(z: torch.Tensor, col: int, E: int,
+                 correction: Optional[torch.Tensor], top: int):
+    """Scores s = softmax of the fp32 logits z[:, col:col + E] over all of
+    them; the ``top`` largest s + correction are chosen (the lower index
+    wins a tie) and weighted by their s, not renormalised. Returns (weights
+    [T, top] fp32, indices [T, top] int32)."""
+    assert z.dtype == torch.float32
+    if z.is_cuda:
+        wt, idx = _ext().moe_route_scores(z.contiguous(), int(col), int(E),
+                                          correction, int(top))
+        return wt, idx
+    s = torch.softmax(z[:, col:col + E], -1)
+    c = s if correction is None else s + correction
+    idx = torch.sort(c, dim=-1, descending=True, stable=True).indices[:, :top]
+    return s.gather(1, idx), idx.to(torch.int32)
+
+
 def expert_gated_ff(h: torch.Tensor, wts: torch.Tensor, idx: torch.Tensor,
-                    gate_up: torch.Tensor, down: torch.Tensor, act: str, *,
+                    gate_up: torch.Tensor, down: torch.Tensor, act, *,
                     shared: Optional[torch.Tensor] = None,
                     sgate: Optional[torch.Tensor] = None,
-                    sgate_col: int = 0) -> torch.Tensor:
+                    sgate_col: int = 0, identity: int = 0) -> torch.Tensor:
     """sum_j wts[:, j] E_idx[:, j](h), E_e(x) = down_e(act(gate_e x) *
-    (up_e x)), plus ``shared`` [T, W] times sigmoid(sgate[:, sgate_col]).
-    gate_up [E, 2 ff, W] and down [E, W, ff] are the stacked experts; their
-    products run in h's dtype with fp32 accumulation, the weighted sum is
-    fp32; result in h's dtype."""
+    (up_e x)) (``act`` as for :func:`act_gate`), plus ``shared`` [T, W]
+    times sigmoid(sgate[:, sgate_col]). gate_up [E, 2 ff, W] and down
+    [E, W, ff] are the stacked experts; their products run in h's dtype with
+    fp32 accumulation, the weighted sum is fp32; result in h's dtype.
+    Indices E .. E + ``identity`` - 1 are identity experts: E_e(x) = x."""
     T, W = h.shape
     E = gate_up.shape[0]
     if h.is_cuda:
+        code, limit, alpha = _act_code(act)
         return _ext().moe_experts(h.contiguous(), wts, idx, gate_up, down,
-                                  GATE_ACTS[act], shared, sgate,
-                                  int(sgate_col))
+                                  code, limit, alpha, int(identity), shared,
+                                  sgate, int(sgate_col))
     out = torch.zeros(T, W, dtype=torch.float32)
+    if identity:
+        out += h.float() * (wts * (idx >= E)).sum(-1, keepdim=True)
     for e in range(E):
         tok, choice = (idx == e).nonzero(as_tuple=True)
         if tok.numel() == 0:
@@ -1220,3 +1274,126 @@ def expert_gated_ff(h: torch.Tensor, wts: torch.Tensor, idx: torch.Tensor,
                 sgate[:, sgate_col:sgate_col + 1].float())
         out += s
     return out.to(h.dtype)
+
+
+# ---------------------------------------------------------------------------
+# gated delta rule, bigram embedding, thin fp32 projections
+# ---------------------------------------------------------------------------
+def delta_chunk(D: int) -> int:
+    """Tokens per chunk of the chunk form of the gated delta rule for key
+    size D; 0 if the chunk kernels do not serve it."""
+    return 64 if D <= 64 else 32 if D <= 256 else 0
+
+
+def delta_scan(x: torch.Tensor, offs, proj: torch.Tensor, r_off: int,
+               b: torch.Tensor, b_off: int, a2t: torch.Tensor,
+               dt_bias: torch.Tensor, A_log: torch.Tensor, S: torch.Tensor,
+               meta: RaggedMeta, H: int, G: int, D: int,
+               V: int) -> torch.Tensor:
+    """Gated delta rule per head: S <- diag(g) S; u = beta (v - S^T k);
+    S <- S + k u^T; o = S^T q.
+
+    x [T, *] fp32 holds q [G*D] | k [G*D] | v [H*V] at columns ``offs``; q
+    and k of head h are those of group floor(h / (H/G)), made unit vectors
+    x / sqrt(sum x^2 + 1e-6), q also times D^-1/2. beta = sigmoid of
+    b[:, b_off + h] (fp32). g = exp(-exp(A_log_h) softplus(z)) with
+    z = r a2t + dt_bias, r [R] = columns of proj from ``r_off``; a2t
+    [R, H*D], dt_bias [H*D], A_log [H] fp32. The state pool S
+    [slots, H, D, V] (fp32) is read at ``meta.slots`` (zeros for a sequence
+    with no cached tokens) and written back. Everything is fp32; returns the
+    raw read-out [T, H*V]."""
+    q_off, k_off, v_off = (int(c) for c in offs)
+    T, R = x.shape[0], a2t.shape[0]
+    assert x.dtype == b.dtype == S.dtype == torch.float32
+    assert a2t.dtype == dt_bias.dtype == A_log.dtype == torch.float32
+    if x.is_cuda:
+        C = delta_chunk(D)
+        args = (x, q_off, k_off, v_off, proj, int(r_off), b, int(b_off), a2t,
+                dt_bias, A_log, S)
+        if (C and max(meta.new_h) >= 2 * C
+                and not os.environ.get("TL_NO_SCAN_CHUNKS")
+                and T * H * (3 * D + C + V) * 4 <= (1 << 33)
+                and _ext().delta_chunks_ok(int(D), int(R), C)):
+            # long prompt portions: per-chunk factors in parallel, then the
+            # chain over a sequence's chunks
+            cu_c, _, _, base, cnt, nc, _ = meta.scan_chunks(C)
+            return _ext().delta_chunks(*args, cu_c, base, cnt, meta.slots,
+                                       meta.pos0, int(H), int(G), int(D),
+                                       int(V), int(C))
+        return _ext().delta_scan(*args, meta.cu, meta.slots, meta.pos0,
+                                 int(H), int(G), int(D), int(V))
+    F = torch.nn.functional
+    rep = H // G
+
+    def unit(c):
+        u = x[:, c:c + G * D].view(T, G, D)
+        u = u / torch.sqrt((u * u).sum(-1, keepdim=True) + 1e-6)
+        return u.repeat_interleave(rep, 1)
+
+    q, k = unit(q_off) * D ** -0.5, unit(k_off)
+    v = x[:, v_off:v_off + H * V].view(T, H, V)
+    beta = torch.sigmoid(b[:, b_off:b_off + H])
+    z = F.softplus(proj[:, r_off:r_off + R].float() @ a2t + dt_bias)
+    g = torch.exp(-torch.exp(A_log).view(1, H, 1) * z.view(T, H, D))
+    o = torch.empty(T, H, V)
+    for s in range(meta.B):
+        t0, t1 = meta.cu_h[s], meta.cu_h[s + 1]
+        if t1 == t0:
+            continue
+        slot = meta.slots_h[s]
+        Sb = (torch.zeros(H, D, V) if meta.pos0_h[s] == 0
+              else S[slot].clone())
+        for t in range(t0, t1):
+            Sb = g[t].unsqueeze(-1) * Sb
+            u = beta[t].unsqueeze(-1) * (
+                v[t] - (Sb * k[t].unsqueeze(-1)).sum(1))
+            Sb = Sb + k[t].unsqueeze(-1) * u.unsqueeze(1)
+            o[t] = (Sb * q[t].unsqueeze(-1)).sum(1)
+        S[slot] = Sb
+    return o.reshape(T, H * V)
+
+
+def bigram_embed(tokens: torch.Tensor, embed: torch.Tensor,
+                 table: torch.Tensor, prev: torch.Tensor, meta: RaggedMeta,
+                 mul_prev: int, mul_cur: int) -> torch.Tensor:
+    """fp32 [T, W]: embed[token] + table[row] with row = (previous token *
+    mul_prev + token * mul_cur) mod n, n = rows of ``table`` - 1, and row n
+    for a sequence's first token. ``prev`` [slots] int32 holds the token
+    before a portion and is left holding the portion's last one."""
+    tokens = tokens.reshape(-1).long()
+    assert prev.dtype == torch.int32 and prev.dim() == 1
+    if tokens.is_cuda:
+        return _ext().bigram_embed(tokens.contiguous(), embed, table, prev,
+                                   meta.tok_seq, meta.cu, meta.slots,
+                                   meta.pos0, int(mul_prev), int(mul_cur))
+    n = table.shape[0] - 1
+    before = torch.roll(tokens, 1)
+    first = torch.zeros(tokens.shape[0], dtype=torch.bool)
+    for b in range(meta.B):
+        t0, t1 = meta.cu_h[b], meta.cu_h[b + 1]
+        if t1 == t0:
+            continue
+        if meta.pos0_h[b] == 0:
+            first[t0] = True
+        else:
+            before[t0] = int(prev[meta.slots_h[b]])
+        prev[meta.slots_h[b]] = int(tokens[t1 - 1])
+    rows = torch.where(first, torch.full_like(tokens, n),
+                       (before * int(mul_prev) + tokens * int(mul_cur)) % n)
+    return embed[tokens].float() + table[rows].float()
+
+
+def thin_linear(h: torch.Tensor, w: torch.Tensor,
+                bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """h w^T + bias with fp32 results for a projection to few outputs (gate
+    and step-size pre-activations, router logits): h [T, W] and w [N, W] in
+    the serving dtype, products accumulated and returned in fp32; bias fp32
+    [N]."""
+    if h.is_cuda:
+        if h.shape[0] <= 64:
+            return _ext().thin_linear(h.contiguous(), w, bias)
+        z = (h @ w.t() if h.dtype == torch.float32
+             else torch.mm(h, w.t(), out_dtype=torch.float32))
+    else:
+        z = h.float() @ w.float().t()
+    return z if bias is None else z.add_(bias)
