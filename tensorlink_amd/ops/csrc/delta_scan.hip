@@ -52,6 +52,10 @@ constexpr int VT = 64;              // value columns per block of the scan
 constexpr int CT = 32;              // value columns per block of the chain
 constexpr int CS = CT + 4;          // their LDS row stride
 constexpr float LOG_RANGE = 60.f;   // e^60 * e^60 is inside fp32
+// chunk form: a token's log decay is cut here. e^-60 of a memory is nothing
+// beside what any token writes, and the running sums, whose differences are
+// taken, keep their digits.
+constexpr float LOG_FLOOR = -60.f;
 
 using f32x4 = __attribute__((ext_vector_type(4))) float;
 
@@ -361,7 +365,8 @@ __global__ __launch_bounds__(BLOCK) void delta_chunk_prep_kernel(
     float run = 0.f;
 #pragma unroll
     for (int t = 0; t < 16; ++t) {
-      if (d < D && a * 16 + t < n) run += ea * softplus_f(z[t]);
+      if (d < D && a * 16 + t < n)
+        run += fmaxf(ea * softplus_f(z[t]), LOG_FLOOR);
       L[(a * 16 + t) * LS + d] = run;
     }
     tot[a * LS + d] = run;
