@@ -51,13 +51,14 @@ def parse_args():
                    help="layered mode: comma list of size presets")
     p.add_argument("--family",
                    choices=["kepusun", "senulix", "dizepel", "potosun",
-                            "mogisun"],
+                            "mogisun", "lunadra"],
                    default="kepusun",
                    help="layered mode: which layered family to time "
                         "(senulix, dizepel: beside an equal-size dense GQA "
                         "decoder; potosun: beside an equal-size Senulix "
                         "model; mogisun: beside an equal-size Kepusun "
-                        "model)")
+                        "model; lunadra: beside equal-size Kepusun and "
+                        "Mogisun models)")
     p.add_argument("--dp", type=int, default=1,
                    help="data-parallel replicas (train mode; world=dp*pp)")
     return p.parse_args()
@@ -362,6 +363,53 @@ def mogisun_configs(z):
     return mog, kep
 
 
+LUNADRA_SIZES = {
+    # layers: parallel, mlstm, mlstm, parallel, mlstm, parallel
+    "w1024": dict(width=1024, heads=8, kv=2, dim=64, vdim=128, window=1024,
+                  rank=64, experts=16, top=2, ff=320, kep_ff=512,
+                  vocab=32000, batch=8, prompt=2048),
+    "w2048": dict(width=2048, heads=16, kv=4, dim=64, vdim=128, window=1024,
+                  rank=128, experts=32, top=4, ff=512, kep_ff=768,
+                  vocab=32000, batch=8, prompt=2048),
+    "tiny": dict(width=128, heads=2, kv=1, dim=32, vdim=64, window=48,
+                 rank=16, experts=4, top=2, ff=64, kep_ff=96, vocab=512,
+                 batch=2, prompt=96),
+}
+
+
+def lunadra_configs(z):
+    """(Lunadra config, Kepusun config, Mogisun config) of a preset: same
+    width, vocabulary, depth, heads, recurrent state per head, attention key
+    and value width, expert count and top. Lunadra's pairs hold an attention
+    AND a recurrence, so half of its layers do both; Kepusun's two-matrix
+    experts get 3/2 of the width of the gated three-matrix ones."""
+    from tensorlink_amd.models.lunadra import LunadraConfig
+    H, D, V, kv = z["heads"], z["dim"], z["vdim"], z["kv"]
+    mlp = {"kind": "moe", "expert": {"ff": z["ff"], "limit": 7.0},
+           "router": {"experts": z["experts"], "top": z["top"],
+                      "identity": 2},
+           "shared": {"ff": z["ff"], "limit": 7.0}}
+    pa = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": kv, "dim": 2 * D, "vdim": V,
+                 "scale": (2 * D) ** -0.5,
+                 "rot": {"dims": 2 * D, "base": 10000.0},
+                 "mask": {"size": z["window"]}},
+        "right": {"heads": H, "kv_heads": H, "dim": D, "vdim": V, "conv": 4,
+                  "decay_rank": z["rank"], "gate_rank": z["rank"]},
+        "left_scale": 0.7, "right_scale": 0.7}}
+    ma = {"type": "mlstm", "mlp": mlp,
+          "mixer": {"heads": H, "dim": D, "vdim": V, "gate_cap": 15.0}}
+    lun = LunadraConfig.from_dict({
+        "architecture": "Lunadra", "vocab": z["vocab"], "width": z["width"],
+        "norm": {"eps": 1e-6}, "residual_mult": 0.5,
+        "embedding": {"bigram": {"buckets": z["vocab"], "mul_prev": 31,
+                                 "mul_cur": 17}},
+        "layers": [pa, ma, ma, pa, ma, pa]},
+        name="lunadra-" + str(z["width"]))
+    mog, kep = mogisun_configs(dict(z, rank=16))
+    return lun, kep, mog
+
+
 @torch.no_grad()
 def run_layered(args, device, use_gpu):
     """Prefill and decode tokens/s of the Kepusun family beside the
@@ -411,7 +459,14 @@ def run_layered(args, device, use_gpu):
         return out
 
     for name in args.sizes.split(","):
-        if args.family == "mogisun":
+        if args.family == "lunadra":
+            z = LUNADRA_SIZES[name]
+            B, S = z["batch"], z["prompt"]
+            only = os.environ.get("TL_BENCH_ONLY")     # profile one model
+            res = {k: measure(c, B, S) for k, c in zip(
+                ("lunadra", "kepusun", "mogisun"), lunadra_configs(z))
+                if only in (None, k)}
+        elif args.family == "mogisun":
             z = MOGISUN_SIZES[name]
             mog, kep = mogisun_configs(z)
             B, S = z["batch"], z["prompt"]

@@ -21,6 +21,17 @@ int tl_mlstm_seq(const void* proj, int ld, int q_off, int k_off, int v_off,
                  const void* pos0, void* out, int B, int H, int D, int V,
                  float cap, float qscale, float eps, void* F, int summary,
                  int is_f32, hipStream_t stream);
+int tl_mlstm_chunk_tokens();
+int tl_mlstm_chunks_ok(int D, int V, int ld, int q_off, int k_off, int v_off,
+                       int g_off);
+int tl_mlstm_chunks(const void* proj, int ld, int q_off, int k_off,
+                    int v_off, int g_off, const void* gates, int ldg,
+                    const void* norm_w, void* S, void* n, void* m, void* U,
+                    void* nU, void* sc, const void* cu_c, int NC,
+                    const void* base, const void* cnt, const void* slots,
+                    const void* pos0, int B, void* out, int H, int D, int V,
+                    float cap, float qscale, float eps, int is_f32,
+                    hipStream_t stream);
 int tl_mlstm_chain(void* S_tmp, void* n_tmp, void* m_tmp, const void* F_tmp,
                    void* S, void* n, void* m, const void* chunk_base,
                    const void* n_chunks, const void* slots, const void* pos0,
@@ -132,28 +143,25 @@ Tensor relu_sq(Tensor x) {
   return out;
 }
 
-Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
-                 int64_t g_off, Tensor gates, Tensor norm_w, Tensor S,
-                 Tensor n, Tensor m, Tensor cu, Tensor slots, Tensor pos0,
-                 int64_t H, int64_t D, int64_t V, double cap, double qscale,
-                 double eps, c10::optional<Tensor> F_sum) {
-  // F_sum given = summary mode: every ragged entry is run from the empty
-  // state, no output is produced, its slot receives the entry's summary
-  // and F_sum [slots, H] the sum of its log forget gates
+// shapes that the proj / gates / state arguments of the recurrence share
+void check_mlstm(const Tensor& proj, int64_t q_off, int64_t k_off,
+                 int64_t v_off, int64_t g_off, const Tensor& gates,
+                 const Tensor& norm_w, const Tensor& S, const Tensor& n,
+                 const Tensor& m, const Tensor& slots, const Tensor& pos0,
+                 int64_t H, int64_t D, int64_t V) {
   MIX_IN(proj);
   MIX_F32(gates);
   MIX_F32(norm_w);
   MIX_F32(S);
   MIX_F32(n);
   MIX_F32(m);
-  MIX_I32(cu);
   MIX_I32(slots);
   MIX_I32(pos0);
   TORCH_CHECK(proj.dim() == 2, "proj must be [T, L]");
   const int64_t T = proj.size(0), ld = proj.size(1);
-  const int B = slots.size(0);
-  TORCH_CHECK(cu.size(0) == B + 1 && pos0.size(0) == B, "ragged metadata");
-  TORCH_CHECK(q_off + H * D <= ld && k_off + H * D <= ld &&
+  TORCH_CHECK(pos0.size(0) == slots.size(0), "ragged metadata");
+  TORCH_CHECK(q_off >= 0 && k_off >= 0 && v_off >= 0 && g_off >= 0 &&
+                  q_off + H * D <= ld && k_off + H * D <= ld &&
                   v_off + H * V <= ld && g_off + H * V <= ld,
               "projection columns out of range");
   TORCH_CHECK(gates.dim() == 2 && gates.size(0) == T &&
@@ -165,6 +173,22 @@ Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
               "S pool must be [slots, H, D, V]");
   TORCH_CHECK(n.numel() == S.size(0) * H * D && m.numel() == S.size(0) * H,
               "n / m pools do not match S");
+}
+
+Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
+                 int64_t g_off, Tensor gates, Tensor norm_w, Tensor S,
+                 Tensor n, Tensor m, Tensor cu, Tensor slots, Tensor pos0,
+                 int64_t H, int64_t D, int64_t V, double cap, double qscale,
+                 double eps, c10::optional<Tensor> F_sum) {
+  // F_sum given = summary mode: every ragged entry is run from the empty
+  // state, no output is produced, its slot receives the entry's summary
+  // and F_sum [slots, H] the sum of its log forget gates
+  check_mlstm(proj, q_off, k_off, v_off, g_off, gates, norm_w, S, n, m, slots,
+              pos0, H, D, V);
+  MIX_I32(cu);
+  const int64_t T = proj.size(0), ld = proj.size(1);
+  const int B = slots.size(0);
+  TORCH_CHECK(cu.size(0) == B + 1, "ragged metadata");
   const bool summary = F_sum.has_value();
   if (summary) {
     MIX_F32(F_sum.value());
@@ -182,6 +206,47 @@ Tensor mlstm_seq(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
       summary ? 1 : 0, io_is_f32(proj), mix_stream());
   TORCH_CHECK(rc == 0, "mlstm_seq: head sizes outside the kernel's range "
                        "(dim <= 256, vdim <= 1023)");
+  return out;
+}
+
+int64_t mlstm_chunk_tokens() { return tl_mlstm_chunk_tokens(); }
+
+bool mlstm_chunks_ok(int64_t D, int64_t V, int64_t ld, int64_t q_off,
+                     int64_t k_off, int64_t v_off, int64_t g_off) {
+  return tl_mlstm_chunks_ok((int)D, (int)V, (int)ld, (int)q_off, (int)k_off,
+                            (int)v_off, (int)g_off) != 0;
+}
+
+// chunk form: cu_c [NC + 1] token offsets of the chunks; base / cnt [B] first
+// chunk and chunk count per sequence
+Tensor mlstm_chunks(Tensor proj, int64_t q_off, int64_t k_off, int64_t v_off,
+                    int64_t g_off, Tensor gates, Tensor norm_w, Tensor S,
+                    Tensor n, Tensor m, Tensor cu_c, Tensor base, Tensor cnt,
+                    Tensor slots, Tensor pos0, int64_t H, int64_t D,
+                    int64_t V, double cap, double qscale, double eps) {
+  check_mlstm(proj, q_off, k_off, v_off, g_off, gates, norm_w, S, n, m, slots,
+              pos0, H, D, V);
+  MIX_I32(cu_c);
+  MIX_I32(base);
+  MIX_I32(cnt);
+  const int B = slots.size(0);
+  const int64_t NC = cu_c.numel() - 1, T = proj.size(0);
+  TORCH_CHECK(NC >= 0 && base.numel() == B && cnt.numel() == B,
+              "per-sequence chunk metadata");
+  auto out = torch::empty({T, H * V}, proj.options());
+  if (T == 0 || B == 0 || NC == 0) return out;
+  auto U = torch::empty({NC, H, D, V}, S.options());
+  auto nU = torch::empty({NC, H, D}, S.options());
+  auto sc = torch::empty({5, NC, H}, S.options());
+  const int rc = tl_mlstm_chunks(
+      proj.data_ptr(), (int)proj.size(1), (int)q_off, (int)k_off, (int)v_off,
+      (int)g_off, gates.data_ptr(), (int)gates.size(1), norm_w.data_ptr(),
+      S.data_ptr(), n.data_ptr(), m.data_ptr(), U.data_ptr(), nU.data_ptr(),
+      sc.data_ptr(), cu_c.data_ptr(), (int)NC, base.data_ptr(),
+      cnt.data_ptr(), slots.data_ptr(), pos0.data_ptr(), B, out.data_ptr(),
+      (int)H, (int)D, (int)V, (float)cap, (float)qscale, (float)eps,
+      io_is_f32(proj), mix_stream());
+  TORCH_CHECK(rc == 0, "mlstm_chunks: shape outside the kernels' range");
   return out;
 }
 
@@ -335,6 +400,12 @@ void register_mix_ops(pybind11::module& mod) {
   mod.def("relu_sq", &relu_sq, "relu(x)^2");
   mod.def("mlstm_seq", &mlstm_seq,
           "matrix-memory recurrence over ragged sequences (slot state)");
+  mod.def("mlstm_chunk_tokens", &mlstm_chunk_tokens,
+          "tokens per chunk of the MFMA chunk form");
+  mod.def("mlstm_chunks_ok", &mlstm_chunks_ok,
+          "whether the MFMA chunk form serves a shape");
+  mod.def("mlstm_chunks", &mlstm_chunks,
+          "matrix-memory recurrence, chunk form on fp32 MFMA");
   mod.def("mlstm_chain", &mlstm_chain,
           "chain per-chunk mLSTM summaries into per-chunk start states");
   mod.def("kv_append", &kv_append, "scatter new K/V rows into page pools");

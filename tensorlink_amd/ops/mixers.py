@@ -199,13 +199,26 @@ def mlstm_scan(proj: torch.Tensor, offs, gates: torch.Tensor,
     if proj.is_cuda:
         C = _ext()
         gates = gates.contiguous()
+        chunk = C.mlstm_chunk_tokens()
+        if (max(meta.new_h) >= chunk
+                and not os.environ.get("TL_NO_SCAN_CHUNKS")
+                and (proj.shape[0] // chunk + meta.B) * H * D * V * 4
+                <= (1 << 32)
+                and C.mlstm_chunks_ok(D, V, proj.shape[1], q_off, k_off,
+                                      v_off, g_off)):
+            # long prompt portions: chunk form on the fp32 MFMA
+            cu_c, _, _, base, cnt, _, _ = meta.scan_chunks(chunk)
+            return C.mlstm_chunks(proj, q_off, k_off, v_off, g_off, gates,
+                                  norm_w, S, n, m, cu_c, base, cnt,
+                                  meta.slots, meta.pos0, H, D, V, cap,
+                                  qscale, eps)
         chunk = SCAN_CHUNK
         while max(meta.new_h) * H * D * V * 4 // chunk > (1 << 30):
             chunk *= 2                   # bound the chunk-state scratch
         if (max(meta.new_h) >= 4 * chunk
                 and not os.environ.get("TL_NO_SCAN_CHUNKS")):
-            # long prompt portions: chunk-parallel form. (1) every chunk's
-            # own summary from the empty state, all chunks in parallel;
+            # the same for sizes the MFMA form does not serve: (1) every
+            # chunk's own summary from the empty state, all chunks in parallel;
             # (2) a cheap sequential chain turns summaries into the state
             # BEFORE each chunk and updates the slots; (3) every chunk's
             # read-out from its start state, all chunks in parallel.
