@@ -565,8 +565,14 @@ class WindowAttention(nn.Module, _F32Cache):
                          cache.v[layer_idx], *args[3:])
         return (y, proj, self.side_col) if self.side_cols else y
 
-    def _attend(self, proj, col, meta, kpool, vpool, shared=None):
+    def _rows(self, proj, col, meta, kpool, vpool, shared):
+        """Keys and values of the step's tokens to their page rows; the
+        prepared queries, fp32 [T, H*dim]."""
         fr = self._freqs(proj.device) if self.rot_dims else None
+        if not (self.q_norm is not None or self.unit_norm or self.v_mix
+                or self.q_temp or self.interleaved):
+            return mx.qkv_rope_rows(proj, col, self.H, self.rot_dims, fr,
+                                    meta, kpool, vpool)
         qn = self._f32("q_norm") if self.q_norm is not None else None
         kn = self._f32("k_norm") if self.k_norm is not None else None
         v_col = col + self.q_cols + self.k_cols
@@ -592,8 +598,11 @@ class WindowAttention(nn.Module, _F32Cache):
             mx.norm_rope_rows(proj, v_col, self.G, self.V, meta, pool=vpool,
                               mix_src=first[0], mix_col=first[1],
                               mix_lam=self._f32("vmix").reshape(1))
-        q = mx.norm_rope_rows(proj, col, self.H, self.D, meta, norm_w=qn,
+        return mx.norm_rope_rows(proj, col, self.H, self.D, meta, norm_w=qn,
                               norm_cols=self.q_cols, temp=self.q_temp, **rot)
+
+    def _attend(self, proj, col, meta, kpool, vpool, shared=None):
+        q = self._rows(proj, col, meta, kpool, vpool, shared)
         o = mx.flex_attention(
             q, kpool, vpool, meta, self.H, self.scale, window=self.window,
             sink=self.sink,

@@ -8,7 +8,8 @@
 #include <hip/hip_runtime.h>
 
 extern "C" {
-int tl_delta_chunks_ok(int D, int R, int C);
+int tl_delta_chunk_tokens();
+int tl_delta_chunks_ok(int D, int R);
 int tl_delta_row_pad(int D);
 int tl_delta_col_pad(int V);
 int tl_delta_chunks(const void* x, int ldx, int q_off, int k_off, int v_off,
@@ -18,7 +19,7 @@ int tl_delta_chunks(const void* x, int ldx, int q_off, int k_off, int v_off,
                     void* S, const void* cu_c, int NC, const void* base,
                     const void* cnt, const void* slots, const void* pos0,
                     int B, void* W, void* Q, void* Kt, void* Bm, void* U,
-                    void* dec, void* out, int H, int G, int D, int V, int C,
+                    void* dec, void* out, int H, int G, int D, int V,
                     int is_f32, hipStream_t stream);
 int tl_delta_scan(const void* x, int ldx, int q_off, int k_off, int v_off,
                   const void* proj, int ldr, int r_off, int R, const void* b,
@@ -121,18 +122,20 @@ Tensor delta_scan(Tensor x, int64_t q_off, int64_t k_off, int64_t v_off,
   return out;
 }
 
-bool delta_chunks_ok(int64_t D, int64_t R, int64_t C) {
-  return tl_delta_chunks_ok((int)D, (int)R, (int)C) != 0;
+int64_t delta_chunk_tokens() { return tl_delta_chunk_tokens(); }
+
+bool delta_chunks_ok(int64_t D, int64_t R) {
+  return tl_delta_chunks_ok((int)D, (int)R) != 0;
 }
 
-// cu_c [NC + 1] token offsets of the chunks (<= C tokens each); base / cnt
+// cu_c [NC + 1] token offsets of the chunks; base / cnt
 // [B] first chunk and chunk count per sequence
 Tensor delta_chunks(Tensor x, int64_t q_off, int64_t k_off, int64_t v_off,
                     Tensor proj, int64_t r_off, Tensor b, int64_t b_off,
                     Tensor a2t, Tensor dt_bias, Tensor A_log, Tensor S,
                     Tensor cu_c, Tensor base, Tensor cnt, Tensor slots,
-                    Tensor pos0, int64_t H, int64_t G, int64_t D, int64_t V,
-                    int64_t C) {
+                    Tensor pos0, int64_t H, int64_t G, int64_t D,
+                    int64_t V) {
   check_delta(x, q_off, k_off, v_off, proj, r_off, b, b_off, a2t, dt_bias,
               A_log, S, slots, pos0, H, G, D, V);
   DL_I32(cu_c);
@@ -142,12 +145,12 @@ Tensor delta_chunks(Tensor x, int64_t q_off, int64_t k_off, int64_t v_off,
   const int64_t NC = cu_c.numel() - 1;
   TORCH_CHECK(NC >= 0 && base.numel() == B && cnt.numel() == B,
               "per-sequence chunk metadata");
-  TORCH_CHECK(tl_delta_chunks_ok((int)D, (int)a2t.size(0), (int)C),
+  TORCH_CHECK(tl_delta_chunks_ok((int)D, (int)a2t.size(0)),
               "delta_chunks: shape outside the kernels' range");
   auto out = torch::empty({x.size(0), H * V}, x.options());
   if (x.size(0) == 0 || B == 0 || NC == 0) return out;
   const int64_t DP = tl_delta_row_pad((int)D), VP = tl_delta_col_pad((int)V);
-  const int64_t n = NC * H;
+  const int64_t n = NC * H, C = tl_delta_chunk_tokens();
   auto W = torch::empty({n, C, DP}, x.options());
   auto Q = torch::empty({n, C, DP}, x.options());
   auto Kt = torch::empty({n, DP, C}, x.options());
@@ -163,7 +166,7 @@ Tensor delta_chunks(Tensor x, int64_t q_off, int64_t k_off, int64_t v_off,
       (int)NC, base.data_ptr(), cnt.data_ptr(), slots.data_ptr(),
       pos0.data_ptr(), B, W.data_ptr(), Q.data_ptr(), Kt.data_ptr(),
       Bm.data_ptr(), U.data_ptr(), dec.data_ptr(), out.data_ptr(), (int)H,
-      (int)G, (int)D, (int)V, (int)C, delta_is_f32(proj), delta_stream());
+      (int)G, (int)D, (int)V, delta_is_f32(proj), delta_stream());
   TORCH_CHECK(rc == 0, "delta_chunks: launch refused");
   return out;
 }
@@ -224,6 +227,8 @@ Tensor thin_linear(Tensor h, Tensor w, c10::optional<Tensor> bias) {
 void register_delta_ops(pybind11::module& mod) {
   mod.def("delta_scan", &delta_scan,
           "gated delta rule over ragged sequences (slot state)");
+  mod.def("delta_chunk_tokens", &delta_chunk_tokens,
+          "tokens per chunk of the chunk form");
   mod.def("delta_chunks_ok", &delta_chunks_ok,
           "whether the chunk kernels serve a shape");
   mod.def("delta_chunks", &delta_chunks,

@@ -43,6 +43,11 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        int mix_ld, int mix_col, const void* mix_lam,
                        double temp_coef, double temp_every,
                        hipStream_t stream);
+void tl_qkv_rope_rows(const void* src, int ld, int col, int H, int G, int D,
+                      int V, int rot_dims, const void* freqs,
+                      const void* tok_seq, const void* tok_pos,
+                      const void* table, int P, int T, void* q, void* kpool,
+                      void* vpool, int is_f32, hipStream_t stream);
 int tl_flex_attn_heads_per_block(int H, int G, int DK, int V, int has_talk);
 int tl_flex_attn_rows(const void* q, const void* kpool, const void* vpool,
                       int vld, const void* tok_seq, const void* tok_pos,
@@ -396,6 +401,51 @@ TlFlexExtra flex_extra(int64_t T, int64_t H, int64_t V, int64_t window,
   return ex;
 }
 
+// q | k | v columns of src: q rotated, fp32 [T, H*D]; k (rotated) and v to
+// the tokens' page rows
+Tensor qkv_rope_rows(Tensor src, int64_t col, int64_t H, int64_t rot_dims,
+                     c10::optional<Tensor> freqs, Tensor tok_seq,
+                     Tensor tok_pos, Tensor table, Tensor kpool,
+                     Tensor vpool) {
+  SEQ_IN(src);
+  SEQ_I32(tok_seq);
+  SEQ_I32(tok_pos);
+  SEQ_I32(table);
+  SEQ_IN(kpool);
+  SEQ_IN(vpool);
+  TORCH_CHECK(src.dim() == 2 && kpool.dim() == 4 && vpool.dim() == 4 &&
+                  kpool.size(2) == 128 && vpool.size(2) == 128 &&
+                  kpool.size(1) == vpool.size(1) &&
+                  kpool.scalar_type() == src.scalar_type() &&
+                  vpool.scalar_type() == src.scalar_type(),
+              "pools must be [pages, G, 128, *] in src's dtype");
+  const int64_t T = src.size(0), G = kpool.size(1), D = kpool.size(3),
+                V = vpool.size(3);
+  TORCH_CHECK(col >= 0 && H >= 1 && col + (H + G) * D + G * V <= src.size(1),
+              "columns out of range");
+  TORCH_CHECK(tok_seq.numel() == T && tok_pos.numel() == T && table.dim() == 2,
+              "ragged metadata");
+  TORCH_CHECK(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= D &&
+                  rot_dims <= 8192,
+              "rotated dimensions out of range");
+  if (rot_dims > 0)
+    TORCH_CHECK(freqs.has_value() && freqs->is_cuda() &&
+                    freqs->is_contiguous() &&
+                    freqs->scalar_type() == torch::kDouble &&
+                    freqs->numel() == rot_dims / 2,
+                "freqs must be float64 [rot_dims / 2]");
+  auto q = torch::empty({T, H * D}, src.options().dtype(torch::kFloat));
+  tl_qkv_rope_rows(src.data_ptr(), (int)src.size(1), (int)col, (int)H, (int)G,
+                   (int)D, (int)V, (int)rot_dims,
+                   rot_dims > 0 ? freqs->data_ptr() : nullptr,
+                   tok_seq.data_ptr(), tok_pos.data_ptr(), table.data_ptr(),
+                   (int)table.size(1), (int)T, q.data_ptr(),
+                   kpool.data_ptr(), vpool.data_ptr(), act_is_f32(src),
+                   seq_stream());
+  return q;
+}
+
+
 Tensor flex_attn_rows(Tensor q, Tensor kpool, c10::optional<Tensor> vpool,
                       Tensor tok_seq, Tensor tok_pos, Tensor table,
                       c10::optional<Tensor> talk, int64_t H, double scale,
@@ -661,6 +711,8 @@ void register_seq_ops(pybind11::module& mod) {
   mod.def("gelu_mul", &gelu_mul,
           "GELU (erf or tanh form) times an optional gathered table slice");
   mod.def("soft_cap_", &soft_cap_, "cap * tanh(z / cap) in place");
+  mod.def("qkv_rope_rows", &qkv_rope_rows,
+          "rotate q and k, scatter k and v to page rows, one launch");
   mod.def("norm_rope_rows", &norm_rope_rows,
           "RMS norm (whole range or per head) + rotary positions (halves or "
           "interleaved) + optional blend on projection rows, dense or "

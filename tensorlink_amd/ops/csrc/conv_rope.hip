@@ -176,6 +176,127 @@ __global__ __launch_bounds__(BLOCK) void conv_rope_rows_kernel(
   }
 }
 
+struct alignas(8) bf16x4 {
+  bf16 v[4];
+};
+DEVINLINE void ld4(const float* p, float (&o)[4]) {
+  const float4 x = *reinterpret_cast<const float4*>(p);
+  o[0] = x.x;
+  o[1] = x.y;
+  o[2] = x.z;
+  o[3] = x.w;
+}
+DEVINLINE void ld4(const bf16* p, float (&o)[4]) {
+  const bf16x4 x = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) o[e] = bf2f(x.v[e]);
+}
+
+// The same without rotation and without pools, N, ld and col multiples of 4:
+// a thread owns four channels of a tile, whose rows are all in flight before
+// the first product.
+template <typename T, int K>
+__global__ __launch_bounds__(BLOCK) void conv_dense_kernel(
+    const T* __restrict__ src, int ld, int col, int N,
+    const float* __restrict__ taps, const float* __restrict__ bias,
+    int act_silu, float* __restrict__ hist, const int* __restrict__ tiles,
+    const int* __restrict__ cu, const int* __restrict__ slots,
+    const int* __restrict__ pos0, float* __restrict__ out) {
+  const int c = (blockIdx.y * BLOCK + threadIdx.x) * 4;
+  if (c >= N) return;                // no barrier in this kernel
+  const int seq = tiles[blockIdx.x * 4 + 0];
+  const int tok0 = tiles[blockIdx.x * 4 + 1];
+  const int n = tiles[blockIdx.x * 4 + 2];
+  const int c0 = cu[seq], ntot = cu[seq + 1] - c0;
+  const bool first = tok0 == c0, fresh = pos0[seq] == 0;
+  float* hs = hist + (int64_t)slots[seq] * (K - 1) * N + c;
+  const T* sc = src + col + c;
+  float u[K - 1 + TILE][4];          // rows tok0 - (K-1) .. tok0 + TILE - 1
+#pragma unroll
+  for (int i = 0; i < TILE; ++i)
+    ld4(sc + (int64_t)(tok0 + min(i, n - 1)) * ld, u[K - 1 + i]);
+  if (!first) {                      // TILE >= K - 1: all in the portion
+#pragma unroll
+    for (int j = 0; j < K - 1; ++j)
+      ld4(sc + (int64_t)(tok0 - (K - 1) + j) * ld, u[j]);
+  } else {
+#pragma unroll
+    for (int j = 0; j < K - 1; ++j) {
+      if (fresh) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) u[j][e] = 0.f;
+      } else {
+        ld4(hs + (int64_t)j * N, u[j]);
+      }
+    }
+  }
+  float w[4 * K], b[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int j = 0; j < K; ++j) {
+    float x[4];
+    ld4(taps + (int64_t)c * K + 4 * j, x);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[4 * j + e] = x[e];
+  }
+  if (bias) ld4(bias + c, b);
+#pragma unroll
+  for (int i = 0; i < TILE; ++i) {
+    if (i < n) {
+      float a[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        a[e] = b[e];
+#pragma unroll
+        for (int j = 0; j < K; ++j) a[e] += w[e * K + j] * u[i + j][e];
+        if (act_silu) a[e] = silu_f(a[e]);
+      }
+      *reinterpret_cast<float4*>(out + (int64_t)(tok0 + i) * N + c) =
+          make_float4(a[0], a[1], a[2], a[3]);
+    }
+  }
+  if (!first) return;
+  // the portion's last K-1 rows; a thread reads and writes its own channels
+#pragma unroll
+  for (int r = 0; r < K - 1; ++r) {
+    const int rr = ntot - (K - 1) + r;
+    float v[4] = {0.f, 0.f, 0.f, 0.f};
+    if (rr >= 0)
+      ld4(sc + (int64_t)(c0 + rr) * ld, v);
+    else if (!fresh)   // ascending: source row r + ntot is not overwritten yet
+      ld4(hs + (int64_t)(r + ntot) * N, v);
+    *reinterpret_cast<float4*>(hs + (int64_t)r * N) =
+        make_float4(v[0], v[1], v[2], v[3]);
+  }
+}
+
+template <typename T>
+void launch_dense(const T* src, int ld, int col, int N, const float* taps,
+                  const float* bias, int act_silu, float* hist, int K,
+                  const int* tiles, int n_tiles, const int* cu,
+                  const int* slots, const int* pos0, float* out,
+                  hipStream_t stream) {
+  const dim3 grid(n_tiles, (N / 4 + BLOCK - 1) / BLOCK);
+#define TL_CD(KK)                                                            \
+  case KK:                                                                   \
+    hipLaunchKernelGGL((conv_dense_kernel<T, KK>), grid, dim3(BLOCK), 0,     \
+                       stream, src, ld, col, N, taps, bias, act_silu, hist,  \
+                       tiles, cu, slots, pos0, out);                         \
+    break
+  switch (K) {
+    TL_CD(1);
+    TL_CD(2);
+    TL_CD(3);
+    TL_CD(4);
+    TL_CD(5);
+    TL_CD(6);
+    TL_CD(7);
+    TL_CD(8);
+    default:
+      TL_CD(9);
+  }
+#undef TL_CD
+}
+
 }  // namespace
 
 extern "C" {
@@ -196,6 +317,23 @@ int tl_conv_rope_rows(const void* src, int ld, int col, int n_heads, int D,
     return 1;
   const size_t smem = sizeof(float) * 2 * TILE * (size_t)(rot_dims / 2);
   if (smem > 64 * 1024) return 1;
+  const int N = n_heads * D;
+  if (rot_dims == 0 && pool_heads == 0 && N % 4 == 0 && ld % 4 == 0 &&
+      col % 4 == 0) {
+    if (is_f32)
+      launch_dense<float>((const float*)src, ld, col, N, (const float*)taps,
+                          (const float*)bias, act_silu, (float*)hist, K,
+                          (const int*)tiles, n_tiles, (const int*)cu,
+                          (const int*)slots, (const int*)pos0, (float*)out,
+                          stream);
+    else
+      launch_dense<bf16>((const bf16*)src, ld, col, N, (const float*)taps,
+                         (const float*)bias, act_silu, (float*)hist, K,
+                         (const int*)tiles, n_tiles, (const int*)cu,
+                         (const int*)slots, (const int*)pos0, (float*)out,
+                         stream);
+    return 0;
+  }
   const int items = n_heads * (D - rot_dims / 2);
   const int gy = n_tiles >= 512 ? 1 : min(16, max(1, (items + BLOCK - 1) / BLOCK));
   const dim3 grid(n_tiles, gy);

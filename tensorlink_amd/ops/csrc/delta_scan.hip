@@ -19,8 +19,8 @@
 // and the token loop has no barrier. Key sizes beyond the register budget
 // take the generic kernel (state in the slot's memory).
 //
-// Long prompt portions take the chunk form: chunks of C = 16 * NS tokens in
-// NS tiles of 16. With L_t the running sum of log g inside the chunk,
+// Long prompt portions take the chunk form: chunks of C = 32 tokens in two
+// tiles of 16. With L_t the running sum of log g inside the chunk,
 //     A_ts = beta_t sum_d k_td k_sd e^(L_td - L_sd)               (s < t)
 //     (I + A) U = diag(beta) V - diag(beta) [K e^L] S0
 //     O  = [Q e^L] S0 + B U,  B_ts = sum_d q_td k_sd e^(L_td - L_sd)  (s <= t)
@@ -29,7 +29,7 @@
 // [K e^L] and U0 = (I + A)^-1 diag(beta) V by block forward substitution (the
 // 16 x 16 diagonal blocks are inverted), B, [Q e^L], [K e^(L_C - L)]^T and
 // e^(L_C). tl_delta_chunk_chain then walks a sequence's chunks with
-// U = U0 - W S0; one block per (sequence, head, 32 value columns).
+// U = U0 - W S0; one block per (sequence, head, 16 value columns).
 // Exponents: with l the running sum inside a token's own tile and tot_a a
 // tile's total, products between tiles use e^(l_i + sum of tiles between) and
 // e^(tot_b - l_j), all exponents <= 0. Inside a tile the product factors as
@@ -49,7 +49,8 @@ namespace {
 constexpr int BLOCK = 256;
 constexpr int RT = 8;               // tokens per round of the scan
 constexpr int VT = 64;              // value columns per block of the scan
-constexpr int CT = 32;              // value columns per block of the chain
+constexpr int CHUNK = 32;           // tokens per chunk
+constexpr int CT = 16;              // value columns per block of the chain
 constexpr int CS = CT + 4;          // their LDS row stride
 constexpr float LOG_RANGE = 60.f;   // e^60 * e^60 is inside fp32
 // chunk form: a token's log decay is cut here. e^-60 of a memory is nothing
@@ -131,18 +132,26 @@ __global__ __launch_bounds__(BLOCK) void delta_scan_kernel(
           1.f / (1.f + expf(-p.b[(int64_t)(tb + threadIdx.x) * p.ldb +
                                  p.b_off + h]));
     __syncthreads();
-    // decays, spread over the block
-    for (int i = threadIdx.x; i < nt * 4 * DR; i += BLOCK) {
-      const int tt = i / (4 * DR), d = i - tt * (4 * DR);
-      float a = 1.f;
-      if (d < D) {
-        const int hd = h * D + d;
-        float z = p.dt_bias[hd];
-        for (int r = 0; r < p.R; ++r)
-          z += rs[tt * p.R + r] * p.a2t[(int64_t)r * H * D + hd];
-        a = expf(ea * softplus_f(z));
+    // decays: four lanes per channel, eight loads in flight each
+    for (int i = threadIdx.x; i < nt * 4 * DR * 4; i += BLOCK) {
+      const int j = i & 3, w = i >> 2;
+      const int tt = w / (4 * DR), d = w - tt * (4 * DR);
+      const int hd = h * D + min(d, D - 1);
+      float z = 0.f;
+      for (int r0 = j; r0 < p.R; r0 += 32) {
+        float x[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          x[e] = p.a2t[(int64_t)min(r0 + 4 * e, p.R - 1) * H * D + hd];
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          if (r0 + 4 * e < p.R) z += rs[tt * p.R + r0 + 4 * e] * x[e];
       }
-      gs[tt * DP + (d / DR) * GS + d % DR] = a;
+      z += __shfl_xor(z, 1, WAVE_SIZE);
+      z += __shfl_xor(z, 2, WAVE_SIZE);
+      if (j == 0)
+        gs[tt * DP + (d / DR) * GS + d % DR] =
+            d < D ? expf(ea * softplus_f(z + p.dt_bias[hd])) : 1.f;
     }
     // unit vectors, one wave per token
     for (int tt = wave; tt < nt; tt += BLOCK / WAVE_SIZE) {
@@ -287,20 +296,49 @@ struct DeltaScratch {
   float* U;     // [C][VP]
   float* dec;   // [DP]      e^(L_C)
 };
+// The matrices are cut into 16 x 16 tiles, row tiles first, and a tile is
+// stored in the order the chain's waves hold it, four elements per lane, so
+// that every load is one contiguous KiB: W, Q, Kt and B as A operands (lane
+// (i, g) has row i, columns 4g .. 4g + 3), U as an accumulator (rows 4g ..
+// 4g + 3 of column i).
+DEVINLINE int operand_at(int row, int col) {     // inside a tile
+  return ((col >> 2) * 16 + row) * 4 + (col & 3);
+}
 
-// grid (chunks, H)
+// A barrier for exchanges through LDS only: global loads stay in flight.
+DEVINLINE void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
+DEVINLINE f32x4 mfma4(const float4& a, float b0, float b1, float b2, float b3,
+                      f32x4 c) {
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b0, c, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b1, c, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b2, c, 0, 0, 0);
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b3, c, 0, 0, 0);
+}
+
+// grid (chunks, H). LDS arrays of rows [token][channel]: first the raw q and
+// k and the running logs, then, in place, q e^l, k e^l and k e^(tot - l)
 template <typename T, int NS, int DT>
-__global__ __launch_bounds__(BLOCK) void delta_chunk_prep_kernel(
+__global__ __launch_bounds__(BLOCK, 4) void delta_chunk_prep_kernel(
     const T* __restrict__ proj, DeltaSrc p, const int* __restrict__ cu_c,
     DeltaScratch s, int H, int D, int V, int VP) {
+  static_assert(NS == 2, "no tile lies between two others");
   constexpr int C = 16 * NS, DP = 16 * DT;
   constexpr int LS = DP + 4, AS = C + 4;
   extern __shared__ __align__(16) float lds[];
   __shared__ int far[NS];
   __shared__ float qn[C], kn[C], bt[C];
-  float* L = lds;                  // [C][LS] running logs inside a tile
-  float* tot = L + C * LS;         // [NS][LS]
-  float* A = tot + NS * LS;        // [C][AS]; first the low-rank rows [R][C]
+  float* Qe = lds;                 // [C][LS]
+  float* Ke = Qe + C * LS;
+  float* Kd = Ke + C * LS;         // first L, the running logs inside a tile
+  float* tot = Kd + C * LS;        // [NS][LS] a tile's sum of logs
+  float* Et = tot + NS * LS;       // [NS][LS] e^tot
+  float* Ei = Et + NS * LS;        // [NS][LS] e^(-tot) (tiles in range only)
+  float* A = Ei + NS * LS;        // [C][AS]; first the low-rank rows [C][RS]
   const int ch = blockIdx.x, h = blockIdx.y, hq = h / p.rep;
   const int t0 = cu_c[ch], n = cu_c[ch + 1] - t0;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -310,23 +348,62 @@ __global__ __launch_bounds__(BLOCK) void delta_chunk_prep_kernel(
   const float* vh = p.x + (int64_t)t0 * p.ldx + p.v_off + h * V;
   const int64_t ci = (int64_t)ch * H + h;
 
-  // ---- decays: running sums of log g inside each tile, tile totals
+  // ---- stage: low-rank rows, raw q and k, step sizes
   if (threadIdx.x < NS) far[threadIdx.x] = 0;
-  for (int i = threadIdx.x; i < C * p.R; i += BLOCK) {
-    const int t = i / p.R, r = i - t * p.R;
-    A[r * C + t] =
-        t < n ? ldf<T>(proj + (int64_t)(t0 + t) * p.ldr + p.r_off + r) : 0.f;
+  const int RP = (p.R + 15) / 16 * 16, RS = RP + 4;
+  // (loads are unconditional, from the nearest place that exists, and what
+  // does not exist is cleared afterwards: no branch around a load, so that
+  // all of them are in flight together)
+  {
+    constexpr int TPT = BLOCK / C;   // threads per token
+    const int t = threadIdx.x / TPT, j = threadIdx.x % TPT;
+    const T* row = proj + (int64_t)(t0 + min(t, n - 1)) * p.ldr + p.r_off;
+    for (int r0 = 0; r0 < RP; r0 += TPT * 8) {
+      float x[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        x[e] = ldf<T>(row + min(r0 + e * TPT + j, p.R - 1));
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int r = r0 + e * TPT + j;
+        if (r < RP) A[t * RS + r] = t < n && r < p.R ? x[e] : 0.f;
+      }
+    }
   }
-  // norms and step sizes meanwhile: four tokens per wave and step
+  {
+    constexpr int IT = C * DP / BLOCK;
+    float q[IT], k[IT];
+#pragma unroll
+    for (int i = 0; i < IT; ++i) {
+      const int e = i * BLOCK + threadIdx.x, t = e / DP, d = e - t * DP;
+      const int64_t o = (int64_t)min(t, n - 1) * p.ldx + min(d, D - 1);
+      q[i] = qh[o];
+      k[i] = kh[o];
+    }
+#pragma unroll
+    for (int i = 0; i < IT; ++i) {
+      const int e = i * BLOCK + threadIdx.x, t = e / DP, d = e - t * DP;
+      const bool in = t < n && d < D;
+      Qe[t * LS + d] = in ? q[i] : 0.f;
+      Ke[t * LS + d] = in ? k[i] : 0.f;
+    }
+  }
+  if (threadIdx.x < C)
+    bt[threadIdx.x] =
+        threadIdx.x < n
+            ? 1.f / (1.f + expf(-p.b[(int64_t)(t0 + threadIdx.x) * p.ldb +
+                                     p.b_off + h]))
+            : 0.f;
+  __syncthreads();
+  // ---- norms (four tokens per wave and step) and decays
   for (int t = wave * 4 + quad; t < C; t += 16) {
     float sq = 0.f, sk = 0.f;
-    if (t < n)
-      for (int d = li; d < D; d += 16) {
-        const float q = qh[(int64_t)t * p.ldx + d];
-        const float k = kh[(int64_t)t * p.ldx + d];
-        sq += q * q;
-        sk += k * k;
-      }
+#pragma unroll
+    for (int d = 0; d < DP; d += 16) {
+      const float q = Qe[t * LS + d + li], k = Ke[t * LS + d + li];
+      sq += q * q;
+      sk += k * k;
+    }
 #pragma unroll
     for (int off = 8; off > 0; off >>= 1) {
       sq += __shfl_xor(sq, off, WAVE_SIZE);
@@ -335,111 +412,128 @@ __global__ __launch_bounds__(BLOCK) void delta_chunk_prep_kernel(
     if (li == 0) {
       qn[t] = p.qscale / sqrtf(sq + 1e-6f);
       kn[t] = 1.f / sqrtf(sk + 1e-6f);
-      bt[t] = t < n ? 1.f / (1.f + expf(-p.b[(int64_t)(t0 + t) * p.ldb +
-                                             p.b_off + h]))
-                    : 0.f;
     }
   }
-  __syncthreads();
   const float ea = -expf(p.A_log[h]);
-  for (int i = threadIdx.x; i < NS * DP; i += BLOCK) {
-    const int a = i / DP, d = i - a * DP;
-    const int hd = h * D + d;
-    float z[16];
-    const float bz = d < D ? p.dt_bias[hd] : 0.f;
+  for (int u = wave; u < NS * DT; u += 4) {
+    const int a = u / DT, d = (u - a * DT) * 16 + li;
+    const bool in = d < D;
+    f32x4 z = (f32x4){0.f, 0.f, 0.f, 0.f};
+    const float* rr = A + (a * 16 + li) * RS + quad * 4;
+    // rows beyond R meet zeros of the other operand, channels beyond D are
+    // never used
+    const float* w2 = p.a2t + h * D + min(d, D - 1);
+    const float bz = p.dt_bias[h * D + min(d, D - 1)];
+    for (int r0 = 0; r0 < RP; r0 += 64) {
+      float w[16];
 #pragma unroll
-    for (int t = 0; t < 16; ++t) z[t] = bz;
-    if (d < D)
-      for (int r = 0; r < p.R; ++r) {
-        const float w = p.a2t[(int64_t)r * H * D + hd];
-        const float4* rr = reinterpret_cast<const float4*>(A + r * C + a * 16);
-#pragma unroll
-        for (int t4 = 0; t4 < 4; ++t4) {
-          const float4 x = rr[t4];
-          z[4 * t4 + 0] += w * x.x;
-          z[4 * t4 + 1] += w * x.y;
-          z[4 * t4 + 2] += w * x.z;
-          z[4 * t4 + 3] += w * x.w;
-        }
+      for (int e = 0; e < 16; ++e) {
+        const int r = r0 + (e >> 2) * 16 + quad * 4 + (e & 3);
+        w[e] = w2[(int64_t)min(r, p.R - 1) * H * D];
       }
-    float run = 0.f;
 #pragma unroll
-    for (int t = 0; t < 16; ++t) {
-      if (d < D && a * 16 + t < n)
-        run += fmaxf(ea * softplus_f(z[t]), LOG_FLOOR);
-      L[(a * 16 + t) * LS + d] = run;
+      for (int e = 0; e < 4; ++e)
+        if (r0 + e * 16 < RP) {
+          const float4 x = *reinterpret_cast<const float4*>(rr + r0 + e * 16);
+          z = mfma4(x, w[4 * e], w[4 * e + 1], w[4 * e + 2], w[4 * e + 3], z);
+        }
     }
-    tot[a * LS + d] = run;
-    if (run < -LOG_RANGE) far[a] = 1;      // same value from every writer
+    // running sums over the tile's 16 tokens: four in this lane, then the
+    // lanes of the same channel
+    float run[4], sum = 0.f;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (in && a * 16 + quad * 4 + r < n)
+        sum += fmaxf(ea * softplus_f(z[r] + bz), LOG_FLOOR);
+      run[r] = sum;
+    }
+    float o = __shfl_up(sum, 16, WAVE_SIZE);
+    if (quad >= 1) sum += o;
+    o = __shfl_up(sum, 32, WAVE_SIZE);
+    if (quad >= 2) sum += o;
+    o = __shfl_up(sum, 16, WAVE_SIZE);
+    const float before = quad >= 1 ? o : 0.f;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      Kd[(a * 16 + quad * 4 + r) * LS + d] = before + run[r];
+    if (quad == 3) {
+      tot[a * LS + d] = sum;
+      Et[a * LS + d] = expf(sum);
+      Ei[a * LS + d] = expf(-sum);
+      if (sum < -LOG_RANGE) far[a] = 1;    // same value from every writer
+    }
   }
   __syncthreads();
 
-  // ---- A (strictly lower, times beta) into LDS, B to memory, by tiles
+  // ---- scores: A (strictly lower, times beta) into LDS, B to memory
   float* Bc = s.B + ci * C * C;
-  for (int u = wave; u < NS * NS; u += 4) {
-    const int a = u / NS, b = u - a * NS;
-    f32x4 ak = (f32x4){0.f, 0.f, 0.f, 0.f}, aq = ak;
-    if (b <= a && a * 16 < n) {
-      if (a == b && far[a]) {
-        // strong decay inside the tile: every score on its own
-        const int j = a * 16 + li;
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = a * 16 + quad * 4 + r;
-          float sk = 0.f, sq = 0.f;
-          if (j <= i && i < n)
-            for (int d = 0; d < D; ++d) {
-              const float w = kh[(int64_t)j * p.ldx + d] *
-                              expf(L[i * LS + d] - L[j * LS + d]);
-              sk += kh[(int64_t)i * p.ldx + d] * w;
-              sq += qh[(int64_t)i * p.ldx + d] * w;
-            }
-          const float f = kn[j];
-          ak[r] = sk * f * kn[i];
-          aq[r] = sq * f * qn[i];
-        }
-      } else {
-        const int i = a * 16 + li, j = b * 16 + li;
-        const float fk = kn[i], fq = qn[i], fj = kn[j];
-#pragma unroll 2
-        for (int dt = 0; dt < DT; ++dt) {
-          const int d = dt * 16 + quad * 4;
-          float q[4], ki[4], kj[4];
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const bool in = d + e < D;
-            q[e] = in && i < n ? qh[(int64_t)i * p.ldx + d + e] : 0.f;
-            ki[e] = in && i < n ? kh[(int64_t)i * p.ldx + d + e] : 0.f;
-            kj[e] = in && j < n ? kh[(int64_t)j * p.ldx + d + e] : 0.f;
-          }
-          const float4 x = *reinterpret_cast<const float4*>(L + i * LS + d);
-          const float4 y = *reinterpret_cast<const float4*>(L + j * LS + d);
-          float ei[4] = {x.x, x.y, x.z, x.w};
-          float ej[4] = {-y.x, -y.y, -y.z, -y.w};
-          if (a != b) {
-#pragma unroll
-            for (int e = 0; e < 4; ++e) {
-              ej[e] += tot[b * LS + d + e];
-              for (int m = b + 1; m < a; ++m) ei[e] += tot[m * LS + d + e];
-            }
-          }
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            const float wi = expf(ei[e]), wj = kj[e] * fj * expf(ej[e]);
-            ak = __builtin_amdgcn_mfma_f32_16x16x4f32(ki[e] * fk * wi, wj, ak,
-                                                      0, 0, 0);
-            aq = __builtin_amdgcn_mfma_f32_16x16x4f32(q[e] * fq * wi, wj, aq,
-                                                      0, 0, 0);
-          }
-        }
-      }
-    }
+  auto put = [&](int a, int b, const f32x4& ak, const f32x4& aq) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int i = a * 16 + quad * 4 + r, j = b * 16 + li;
       A[i * AS + j] = j < i ? ak[r] * bt[i] : 0.f;
-      Bc[i * C + j] = j <= i ? aq[r] : 0.f;
+      Bc[(a * NS + b) * 256 + operand_at(quad * 4 + r, li)] =
+          j <= i ? aq[r] : 0.f;
     }
+  };
+  // diagonal tiles of strong decay: every score on its own, while the raw
+  // vectors and the logs are here
+  if (wave < NS && far[wave]) {
+    const int a = wave, j = a * 16 + li;
+    f32x4 ak, aq;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = a * 16 + quad * 4 + r;
+      float sk = 0.f, sq = 0.f;
+      if (j <= i)
+        for (int d = 0; d < D; ++d) {
+          const float w =
+              Ke[j * LS + d] * expf(Kd[i * LS + d] - Kd[j * LS + d]);
+          sk += Ke[i * LS + d] * w;
+          sq += Qe[i * LS + d] * w;
+        }
+      ak[r] = sk * kn[j] * kn[i];
+      aq[r] = sq * kn[j] * qn[i];
+    }
+    put(a, a, ak, aq);
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < C * DP; i += BLOCK) {
+    const int t = i / DP, o = t * LS + (i - t * DP);
+    const int tt = (t >> 4) * LS + (i - t * DP);
+    const float l = Kd[o], k = Ke[o] * kn[t];
+    const float el = __expf(l), ed = __expf(tot[tt] - l);
+    Qe[o] *= qn[t] * el;
+    Ke[o] = k * el;
+    Kd[o] = k * ed;
+  }
+  __syncthreads();
+  for (int u = wave; u < NS * NS; u += 4) {
+    const int a = u / NS, b = u - a * NS;
+    if (a == b && far[a]) continue;
+    f32x4 ak = (f32x4){0.f, 0.f, 0.f, 0.f}, aq = ak;
+    if (b <= a && a * 16 < n) {
+      const float* qi = Qe + (a * 16 + li) * LS + quad * 4;
+      const float* ki = Ke + (a * 16 + li) * LS + quad * 4;
+      const float* kj = Kd + (b * 16 + li) * LS + quad * 4;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        const float4 q = *reinterpret_cast<const float4*>(qi + dt * 16);
+        const float4 k = *reinterpret_cast<const float4*>(ki + dt * 16);
+        float4 y = *reinterpret_cast<const float4*>(kj + dt * 16);
+        if (a == b) {                // inside a tile e^(-l) alone
+          const float4 e = *reinterpret_cast<const float4*>(
+              Ei + a * LS + dt * 16 + quad * 4);
+          y.x *= e.x;
+          y.y *= e.y;
+          y.z *= e.z;
+          y.w *= e.w;
+        }
+        ak = mfma4(k, y.x, y.y, y.z, y.w, ak);
+        aq = mfma4(q, y.x, y.y, y.z, y.w, aq);
+      }
+    }
+    put(a, b, ak, aq);
   }
   __syncthreads();
 
@@ -469,95 +563,102 @@ __global__ __launch_bounds__(BLOCK) void delta_chunk_prep_kernel(
   for (int u = wave; u < DT + VP / 16; u += 4) {
     const bool isw = u < DT;
     const int col = (isw ? u : u - DT) * 16 + li;
+    float v0[NS][4];
+    if (!isw) {
+#pragma unroll
+      for (int a = 0; a < NS; ++a)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          v0[a][r] = vh[(int64_t)min(a * 16 + quad * 4 + r, n - 1) * p.ldx +
+                        min(col, V - 1)];
+    }
     f32x4 X[NS];
-    float before = 0.f;              // sum of the earlier tiles' logs
 #pragma unroll
     for (int a = 0; a < NS; ++a) {
       f32x4 y;
+      const float eb = isw && a ? Et[col] : 1.f;     // the tile before
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = a * 16 + quad * 4 + r;
         float v = 0.f;
-        if (i < n) {
-          if (isw) {
-            if (col < D)
-              v = kh[(int64_t)i * p.ldx + col] * kn[i] *
-                  expf(before + L[i * LS + col]);
-          } else if (col < V) {
-            v = vh[(int64_t)i * p.ldx + col];
-          }
-        }
-        y[r] = v * bt[i];
+        if (isw) v = Ke[i * LS + col] * eb;
+        else v = col < V ? v0[a][r] : 0.f;
+        y[r] = v * bt[i];            // 0 beyond the chunk's tokens
       }
-      if (isw) before += tot[a * LS + col];
+#pragma unroll
       for (int b = 0; b < a; ++b) {
         const float4 f = *reinterpret_cast<const float4*>(
             A + (a * 16 + li) * AS + b * 16 + quad * 4);
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(-f.x, X[b][0], y, 0, 0, 0);
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(-f.y, X[b][1], y, 0, 0, 0);
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(-f.z, X[b][2], y, 0, 0, 0);
-        y = __builtin_amdgcn_mfma_f32_16x16x4f32(-f.w, X[b][3], y, 0, 0, 0);
+        y = mfma4(f, -X[b][0], -X[b][1], -X[b][2], -X[b][3], y);
       }
       const float4 f = *reinterpret_cast<const float4*>(
           A + (a * 16 + li) * AS + a * 16 + quad * 4);
-      f32x4 z = (f32x4){0.f, 0.f, 0.f, 0.f};
-      z = __builtin_amdgcn_mfma_f32_16x16x4f32(f.x, y[0], z, 0, 0, 0);
-      z = __builtin_amdgcn_mfma_f32_16x16x4f32(f.y, y[1], z, 0, 0, 0);
-      z = __builtin_amdgcn_mfma_f32_16x16x4f32(f.z, y[2], z, 0, 0, 0);
-      z = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w, y[3], z, 0, 0, 0);
+      const f32x4 z = mfma4(f, y[0], y[1], y[2], y[3],
+                            (f32x4){0.f, 0.f, 0.f, 0.f});
       X[a] = z;
+      if (isw) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int i = a * 16 + quad * 4 + r;
-        if (isw) Wc[i * DP + col] = z[r];
-        else Uc[i * VP + col] = z[r];
+        for (int r = 0; r < 4; ++r)
+          Wc[(a * DT + u) * 256 + operand_at(quad * 4 + r, li)] = z[r];
+      } else {
+        *reinterpret_cast<float4*>(
+            Uc + ((a * (VP / 16) + u - DT) * 64 + lane) * 4) =
+            make_float4(z[0], z[1], z[2], z[3]);
       }
     }
   }
 
   // ---- q e^L, (k e^(L_C - L))^T and e^(L_C)
   float* Qc = s.Q + ci * C * DP;
-  for (int i = threadIdx.x; i < C * DP; i += BLOCK) {
-    const int t = i / DP, d = i - t * DP, a = t >> 4;
-    float v = 0.f;
-    if (t < n && d < D) {
-      float e = L[t * LS + d];
-      for (int m = 0; m < a; ++m) e += tot[m * LS + d];
-      v = qh[(int64_t)t * p.ldx + d] * qn[t] * expf(e);
+#pragma unroll
+  for (int u = wave; u < NS * DT; u += 4) {
+    const int a = u / DT, d = (u - a * DT) * 16 + quad * 4;
+    float4 x = *reinterpret_cast<const float4*>(Qe + (a * 16 + li) * LS + d);
+    if (a) {
+      const float4 e = *reinterpret_cast<const float4*>(Et + d);
+      x.x *= e.x;
+      x.y *= e.y;
+      x.z *= e.z;
+      x.w *= e.w;
     }
-    Qc[i] = v;
+    *reinterpret_cast<float4*>(Qc + (u * 64 + lane) * 4) = x;
   }
   float* Kc = s.Kt + ci * C * DP;
-  for (int i = threadIdx.x; i < C * DP; i += BLOCK) {
-    const int d = i / C, t = i - d * C, a = t >> 4;
-    float v = 0.f;
-    if (t < n && d < D) {
-      float e = tot[a * LS + d] - L[t * LS + d];
-      for (int m = a + 1; m < NS; ++m) e += tot[m * LS + d];
-      v = kh[(int64_t)t * p.ldx + d] * kn[t] * expf(e);
-    }
-    Kc[i] = v;
-  }
-  for (int d = threadIdx.x; d < DP; d += BLOCK) {
-    float e = 0.f;
 #pragma unroll
-    for (int m = 0; m < NS; ++m) e += tot[m * LS + d];
-    s.dec[ci * DP + d] = expf(e);
+  for (int u = wave; u < NS * DT; u += 4) {
+    const int dt = u / NS, a = u - dt * NS, d = dt * 16 + li;
+    const float e = a == 0 ? Et[LS + d] : 1.f;
+    const float* kp = Kd + (a * 16 + quad * 4) * LS + d;
+    *reinterpret_cast<float4*>(Kc + (u * 64 + lane) * 4) = make_float4(
+        kp[0] * e, kp[LS] * e, kp[2 * LS] * e, kp[3 * LS] * e);
   }
+  for (int d = threadIdx.x; d < DP; d += BLOCK)
+    s.dec[ci * DP + d] = Et[d] * Et[LS + d];
 }
 
-// grid (B * H, VP / CT): blocks of one (sequence, head) are B * H apart, so
-// with B * H a multiple of 8 they share an XCD's L2
-template <int NS, int DT>
+// what one wave reads of a chunk's scratch
+template <int NS, int DT, int NK>
+struct ChainFrag {
+  float4 wq[DT];                     // its token tile's rows of W or Q
+  float4 u0;
+  float4 b[NS];
+  float4 kt[NK][NS], dec[NK];        // rows of Kt of its state tiles
+  int t0, n;                         // the chunk's tokens
+};
+
+// grid (B * H, VP / CT), 4 waves: blocks of one (sequence, head) are B * H
+// apart, so with B * H a multiple of 8 they share an XCD's L2. Waves 0 and 1
+// compute U = U0 - W S0, waves 2 and 3 the outputs; all update the state. The
+// next chunks' scratch is loaded while a chunk is computed (AHEAD of them).
+template <int DT, int AHEAD>
 __global__ __launch_bounds__(BLOCK) void delta_chunk_chain_kernel(
     DeltaScratch s, const int* __restrict__ cu_c, float* __restrict__ S,
     const int* __restrict__ chunk_base, const int* __restrict__ n_chunks,
     const int* __restrict__ slots, const int* __restrict__ pos0,
     float* __restrict__ out, int H, int D, int V, int VP) {
-  constexpr int C = 16 * NS, DP = 16 * DT;
-  // units of work per wave: token tile x column tile (NS * 2 over 4 waves),
-  // state row tile x column tile (DT * 2 over 4 waves)
-  constexpr int NU = NS * 2 / 4, NW = DT * 2 / 4;
+  constexpr int NS = 2, C = 16 * NS, DP = 16 * DT;
+  constexpr int NW = DT >= 4 ? DT / 4 : 1;     // state row tiles per wave
+  using Frag = ChainFrag<NS, DT, NW>;
   __shared__ __align__(16) float Ss[DP * CS];
   __shared__ __align__(16) float Us[C * CS];
   const int b = blockIdx.x / H, h = blockIdx.x - b * H;
@@ -566,127 +667,158 @@ __global__ __launch_bounds__(BLOCK) void delta_chunk_chain_kernel(
   const int c0 = blockIdx.y * CT;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int li = lane & 15, quad = lane >> 4;
+  const bool is_u = wave < 2;
+  const int ta = wave & 1;           // token tile
+  const bool has_st = wave * NW < DT;
+  const int dt0 = has_st ? wave * NW : 0;           // first state row tile
+  const int c = c0 + li;             // this lane's value column
   float* Sh = S + ((int64_t)slots[b] * H + h) * D * V;
   const bool fresh = pos0[b] == 0;
   f32x4 st[NW];
+  if (has_st)
 #pragma unroll
-  for (int i = 0; i < NW; ++i) {
-    const int w = wave * NW + i, dt = w >> 1, x = w & 1;
-    const int c = c0 + x * 16 + li;
+    for (int i = 0; i < NW; ++i)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int d = dt * 16 + quad * 4 + r;
-      const float v =
-          !fresh && d < D && c < V ? Sh[(int64_t)d * V + c] : 0.f;
-      st[i][r] = v;
-      Ss[d * CS + x * 16 + li] = v;
-    }
-  }
-  __syncthreads();
+      for (int r = 0; r < 4; ++r) {
+        const int d = (dt0 + i) * 16 + quad * 4 + r;
+        const float v =
+            !fresh && d < D && c < V ? Sh[(int64_t)d * V + c] : 0.f;
+        st[i][r] = v;
+        Ss[d * CS + li] = v;
+      }
   const int cb = chunk_base[b];
-  for (int k = 0; k < nc; ++k) {
-    const int ch = cb + k;
-    const int64_t ci = (int64_t)ch * H + h;
-    const int t0 = cu_c[ch], n = cu_c[ch + 1] - t0;
-    // ---- U = U0 - W S0 and the carried part of the outputs
-    f32x4 uo[NU], oo[NU];
+  const float* WQ = is_u ? s.W : s.Q;
+  auto load = [&](Frag& f, int k) {
+    k = min(k, nc - 1);
+    const int64_t ci = (int64_t)(cb + k) * H + h;
+    f.t0 = cu_c[cb + k];
+    f.n = cu_c[cb + k + 1] - f.t0;
+    const float* wq = WQ + ci * C * DP + (ta * DT * 64 + lane) * 4;
 #pragma unroll
-    for (int i = 0; i < NU; ++i) {
-      const int w = wave * NU + i, a = w >> 1, x = w & 1;
-      const float* U0 = s.U + (ci * C + a * 16 + quad * 4) * VP + c0 +
-                        x * 16 + li;
+    for (int dt = 0; dt < DT; ++dt)
+      f.wq[dt] = *reinterpret_cast<const float4*>(wq + dt * 256);
+    // (waves 2 and 3 load what they do not use: no branch around a load)
+    f.u0 = *reinterpret_cast<const float4*>(
+        s.U + ci * C * VP + ((ta * (VP / 16) + blockIdx.y) * 64 + lane) * 4);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) uo[i][r] = U0[(int64_t)r * VP];
-      oo[i] = (f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < NW; ++i) {
+      const float* kp = s.Kt + ci * C * DP +
+                        ((dt0 + i) * NS * 64 + lane) * 4;
+#pragma unroll
+      for (int bb = 0; bb < NS; ++bb)
+        f.kt[i][bb] = *reinterpret_cast<const float4*>(kp + bb * 256);
+      f.dec[i] = *reinterpret_cast<const float4*>(
+          s.dec + ci * DP + (dt0 + i) * 16 + quad * 4);
     }
+    const float* bp = s.B + ci * C * C + (ta * NS * 64 + lane) * 4;
+#pragma unroll
+    for (int bb = 0; bb < NS; ++bb)
+      f.b[bb] = *reinterpret_cast<const float4*>(bp + bb * 256);
+  };
+  auto step = [&](const Frag& f) {
+    // ---- W S0 or Q S0, as two sums
+    f32x4 p0 = (f32x4){0.f, 0.f, 0.f, 0.f}, p1 = p0;
+    float sv[DT][4];
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        sv[dt][e] = Ss[(dt * 16 + quad * 4 + e) * CS + li];
+    __builtin_amdgcn_sched_barrier(0);   // all reads before the products
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
+      if (dt & 1)
+        p1 = mfma4(f.wq[dt], sv[dt][0], sv[dt][1], sv[dt][2], sv[dt][3], p1);
+      else
+        p0 = mfma4(f.wq[dt], sv[dt][0], sv[dt][1], sv[dt][2], sv[dt][3], p0);
+    }
+    f32x4 o = p0 + p1;
+    if (is_u) {
+      float* us = Us + (ta * 16 + quad * 4) * CS + li;
+      us[0] = f.u0.x - o[0];
+      us[CS] = f.u0.y - o[1];
+      us[2 * CS] = f.u0.z - o[2];
+      us[3 * CS] = f.u0.w - o[3];
+    }
+    lds_barrier();
+    float uv[NS][4];
 #pragma unroll
-      for (int i = 0; i < NU; ++i) {
-        const int w = wave * NU + i, a = w >> 1, x = w & 1;
-        const int64_t ro = (ci * C + a * 16 + li) * DP + dt * 16 + quad * 4;
-        const float4 wv = *reinterpret_cast<const float4*>(s.W + ro);
-        const float4 qv = *reinterpret_cast<const float4*>(s.Q + ro);
-        const float* sp = Ss + (dt * 16 + quad * 4) * CS + x * 16 + li;
-        const float s0 = sp[0], s1 = sp[CS], s2 = sp[2 * CS], s3 = sp[3 * CS];
-        uo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(-wv.x, s0, uo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.x, s0, oo[i], 0, 0, 0);
-        uo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(-wv.y, s1, uo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.y, s1, oo[i], 0, 0, 0);
-        uo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(-wv.z, s2, uo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.z, s2, oo[i], 0, 0, 0);
-        uo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(-wv.w, s3, uo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.w, s3, oo[i], 0, 0, 0);
+    for (int bb = 0; bb < NS; ++bb)
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        uv[bb][e] = Us[(bb * 16 + quad * 4 + e) * CS + li];
+    __builtin_amdgcn_sched_barrier(0);
+    // ---- the state after the chunk
+    if (has_st)
+#pragma unroll
+      for (int i = 0; i < NW; ++i) {
+        st[i][0] *= f.dec[i].x;
+        st[i][1] *= f.dec[i].y;
+        st[i][2] *= f.dec[i].z;
+        st[i][3] *= f.dec[i].w;
+#pragma unroll
+        for (int bb = 0; bb < NS; ++bb)
+          st[i] = mfma4(f.kt[i][bb], uv[bb][0], uv[bb][1], uv[bb][2],
+                        uv[bb][3], st[i]);
+        // Ss is read before the barrier above only
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          Ss[((dt0 + i) * 16 + quad * 4 + r) * CS + li] = st[i][r];
       }
-    }
-#pragma unroll
-    for (int i = 0; i < NU; ++i) {
-      const int w = wave * NU + i, a = w >> 1, x = w & 1;
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        Us[(a * 16 + quad * 4 + r) * CS + x * 16 + li] = uo[i][r];
-    }
-    __syncthreads();
     // ---- outputs: the chunk's own part
-#pragma unroll
-    for (int i = 0; i < NU; ++i) {
-      const int w = wave * NU + i, a = w >> 1, x = w & 1;
-      const float* Bp = s.B + (ci * C + a * 16 + li) * C + quad * 4;
+    if (!is_u) {
 #pragma unroll
       for (int bb = 0; bb < NS; ++bb) {
-        if (bb > a) continue;
-        const float4 f = *reinterpret_cast<const float4*>(Bp + bb * 16);
-        const float* up = Us + (bb * 16 + quad * 4) * CS + x * 16 + li;
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.x, up[0], oo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.y, up[CS], oo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.z, up[2 * CS], oo[i], 0, 0, 0);
-        oo[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w, up[3 * CS], oo[i], 0, 0, 0);
+        if (bb > ta) continue;
+        o = mfma4(f.b[bb], uv[bb][0], uv[bb][1], uv[bb][2], uv[bb][3], o);
       }
-      const int c = c0 + x * 16 + li;
       if (c < V)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int t = a * 16 + quad * 4 + r;
-          if (t < n) out[((int64_t)(t0 + t) * H + h) * V + c] = oo[i][r];
+          const int t = ta * 16 + quad * 4 + r;
+          if (t < f.n) out[((int64_t)(f.t0 + t) * H + h) * V + c] = o[r];
         }
     }
-    // ---- the state after the chunk
+    lds_barrier();
+  };
+  lds_barrier();
+  // loads are issued unconditionally (past the end: the last chunk again), so
+  // that their count is known where they are waited for
+  if constexpr (AHEAD == 2) {
+    Frag f0, f1, f2;
+    load(f0, 0);
+    load(f1, 1);
+    for (int k = 0;;) {
+      load(f2, k + 2);
+      step(f0);
+      if (++k >= nc) break;
+      load(f0, k + 2);
+      step(f1);
+      if (++k >= nc) break;
+      load(f1, k + 2);
+      step(f2);
+      if (++k >= nc) break;
+    }
+  } else {
+    Frag f0, f1;
+    load(f0, 0);
+    for (int k = 0;;) {
+      load(f1, k + 1);
+      step(f0);
+      if (++k >= nc) break;
+      load(f0, k + 1);
+      step(f1);
+      if (++k >= nc) break;
+    }
+  }
+  if (has_st)
 #pragma unroll
-    for (int i = 0; i < NW; ++i) {
-      const int w = wave * NW + i, dt = w >> 1, x = w & 1;
-      const float4 de =
-          *reinterpret_cast<const float4*>(s.dec + ci * DP + dt * 16 + quad * 4);
-      st[i][0] *= de.x;
-      st[i][1] *= de.y;
-      st[i][2] *= de.z;
-      st[i][3] *= de.w;
-      const float* Kp = s.Kt + (ci * DP + dt * 16 + li) * C + quad * 4;
+    for (int i = 0; i < NW; ++i)
 #pragma unroll
-      for (int bb = 0; bb < NS; ++bb) {
-        const float4 f = *reinterpret_cast<const float4*>(Kp + bb * 16);
-        const float* up = Us + (bb * 16 + quad * 4) * CS + x * 16 + li;
-        st[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.x, up[0], st[i], 0, 0, 0);
-        st[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.y, up[CS], st[i], 0, 0, 0);
-        st[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.z, up[2 * CS], st[i], 0, 0, 0);
-        st[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(f.w, up[3 * CS], st[i], 0, 0, 0);
+      for (int r = 0; r < 4; ++r) {
+        const int d = (dt0 + i) * 16 + quad * 4 + r;
+        if (d < D && c < V) Sh[(int64_t)d * V + c] = st[i][r];
       }
-      // Ss is read before the barrier above only
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        Ss[(dt * 16 + quad * 4 + r) * CS + x * 16 + li] = st[i][r];
-    }
-    __syncthreads();
-  }
-#pragma unroll
-  for (int i = 0; i < NW; ++i) {
-    const int w = wave * NW + i, dt = w >> 1, x = w & 1;
-    const int c = c0 + x * 16 + li;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int d = dt * 16 + quad * 4 + r;
-      if (d < D && c < V) Sh[(int64_t)d * V + c] = st[i][r];
-    }
-  }
 }
 
 constexpr size_t LDS_MAX = 64 * 1024 - 1024;
@@ -696,48 +828,61 @@ size_t scan_smem(int DR, int R) {
          ((size_t)RT * (3 * 4 * (DR + 4) + VT + 1) + (size_t)RT * R);
 }
 
-size_t prep_smem(int NS, int DT, int R) {
-  const size_t C = 16 * NS, LS = 16 * DT + 4;
-  const size_t a = C * (C + 4), r = C * R;
-  return sizeof(float) * (C * LS + NS * LS + (a > r ? a : r));
+size_t prep_smem(int DT, int R) {
+  const size_t C = CHUNK, NS = CHUNK / 16, LS = 16 * DT + 4;
+  const size_t a = C * (C + 4), r = C * ((R + 15) / 16 * 16 + 4);
+  return sizeof(float) * (3 * C * LS + 3 * NS * LS + (a > r ? a : r));
+}
+
+// LDS a block may have on this device (64 KiB where it is not known)
+size_t lds_limit() {
+  static const size_t lim = [] {
+    int dev = 0, v = 0;
+    if (hipGetDevice(&dev) != hipSuccess ||
+        hipDeviceGetAttribute(&v, hipDeviceAttributeMaxSharedMemoryPerBlock,
+                              dev) != hipSuccess ||
+        v < 64 * 1024)
+      v = 64 * 1024;
+    return (size_t)v - 1024;
+  }();
+  return lim;
 }
 
 // row tiles of 16 that cover D: the sizes the chunk kernels are built for
 int row_tiles(int D) { return D <= 32 ? 2 : D <= 64 ? 4 : D <= 128 ? 8 : 16; }
 
-template <typename T, int NS, int DT>
+template <typename T, int DT, int AHEAD>
 void launch_chunks(const T* proj, const DeltaSrc& p, const int* cu_c, int NC,
                    const int* base, const int* cnt, const int* slots,
                    const int* pos0, int B, float* S, const DeltaScratch& s,
                    float* out, int H, int D, int V, int VP,
                    hipStream_t stream) {
-  hipLaunchKernelGGL((delta_chunk_prep_kernel<T, NS, DT>), dim3(NC, H),
-                     dim3(BLOCK), prep_smem(NS, DT, p.R), stream, proj, p,
-                     cu_c, s, H, D, V, VP);
-  hipLaunchKernelGGL((delta_chunk_chain_kernel<NS, DT>), dim3(B * H, VP / CT),
-                     dim3(BLOCK), 0, stream, s, cu_c, S, base, cnt, slots,
-                     pos0, out, H, D, V, VP);
+  const size_t smem = prep_smem(DT, p.R);
+  if (smem > 64 * 1024)
+    (void)hipFuncSetAttribute(
+        (const void*)delta_chunk_prep_kernel<T, CHUNK / 16, DT>,
+        hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+  hipLaunchKernelGGL((delta_chunk_prep_kernel<T, CHUNK / 16, DT>),
+                     dim3(NC, H), dim3(BLOCK), smem, stream, proj, p, cu_c, s,
+                     H, D, V, VP);
+  hipLaunchKernelGGL((delta_chunk_chain_kernel<DT, AHEAD>),
+                     dim3(B * H, VP / CT), dim3(BLOCK), 0, stream, s, cu_c,
+                     S, base, cnt, slots, pos0, out, H, D, V, VP);
 }
 
 template <typename T>
 void chunks_any(const T* proj, const DeltaSrc& p, const int* cu_c, int NC,
                 const int* base, const int* cnt, const int* slots,
                 const int* pos0, int B, float* S, const DeltaScratch& s,
-                float* out, int H, int D, int V, int VP, int C,
-                hipStream_t stream) {
-#define TL_DC(NS, DT)                                                       \
-  launch_chunks<T, NS, DT>(proj, p, cu_c, NC, base, cnt, slots, pos0, B, S, \
-                           s, out, H, D, V, VP, stream)
+                float* out, int H, int D, int V, int VP, hipStream_t stream) {
+#define TL_DC(DT, AHEAD)                                                     \
+  launch_chunks<T, DT, AHEAD>(proj, p, cu_c, NC, base, cnt, slots, pos0, B, \
+                              S, s, out, H, D, V, VP, stream)
   const int dt = row_tiles(D);
-  if (C == 64) {
-    if (dt <= 2) TL_DC(4, 2);
-    else TL_DC(4, 4);
-  } else {
-    if (dt <= 2) TL_DC(2, 2);
-    else if (dt <= 4) TL_DC(2, 4);
-    else if (dt <= 8) TL_DC(2, 8);
-    else TL_DC(2, 16);
-  }
+  if (dt <= 2) TL_DC(2, 2);
+  else if (dt <= 4) TL_DC(4, 2);
+  else if (dt <= 8) TL_DC(8, 1);
+  else TL_DC(16, 1);
 #undef TL_DC
 }
 
@@ -745,11 +890,12 @@ void chunks_any(const T* proj, const DeltaSrc& p, const int* cu_c, int NC,
 
 extern "C" {
 
-// 1 if the chunk form serves the shape with chunks of C tokens
-int tl_delta_chunks_ok(int D, int R, int C) {
-  if (C != 64 && C != 32) return 0;
-  if (D < 1 || D > 256 || R < 1 || (C == 64 && D > 64)) return 0;
-  return prep_smem(C / 16, row_tiles(D), R) <= LDS_MAX ? 1 : 0;
+int tl_delta_chunk_tokens() { return CHUNK; }
+
+// 1 if the chunk form serves the shape
+int tl_delta_chunks_ok(int D, int R) {
+  if (D < 1 || D > 256 || R < 1) return 0;
+  return prep_smem(row_tiles(D), R) <= lds_limit() ? 1 : 0;
 }
 
 int tl_delta_row_pad(int D) { return 16 * row_tiles(D); }
@@ -764,9 +910,9 @@ int tl_delta_chunks(const void* x, int ldx, int q_off, int k_off, int v_off,
                     void* S, const void* cu_c, int NC, const void* base,
                     const void* cnt, const void* slots, const void* pos0,
                     int B, void* W, void* Q, void* Kt, void* Bm, void* U,
-                    void* dec, void* out, int H, int G, int D, int V, int C,
+                    void* dec, void* out, int H, int G, int D, int V,
                     int is_f32, hipStream_t stream) {
-  if (!tl_delta_chunks_ok(D, R, C) || H <= 0 || V <= 0 || G <= 0 ||
+  if (!tl_delta_chunks_ok(D, R) || H <= 0 || V <= 0 || G <= 0 ||
       H % G != 0)
     return 1;
   if (NC <= 0 || B <= 0) return 0;
@@ -780,12 +926,12 @@ int tl_delta_chunks(const void* x, int ldx, int q_off, int k_off, int v_off,
     chunks_any<float>((const float*)proj, p, (const int*)cu_c, NC,
                       (const int*)base, (const int*)cnt, (const int*)slots,
                       (const int*)pos0, B, (float*)S, s, (float*)out, H, D, V,
-                      VP, C, stream);
+                      VP, stream);
   else
     chunks_any<bf16>((const bf16*)proj, p, (const int*)cu_c, NC,
                      (const int*)base, (const int*)cnt, (const int*)slots,
                      (const int*)pos0, B, (float*)S, s, (float*)out, H, D, V,
-                     VP, C, stream);
+                     VP, stream);
   return 0;
 }
 

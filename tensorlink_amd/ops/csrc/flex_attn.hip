@@ -150,6 +150,62 @@ __global__ __launch_bounds__(BLOCK) void norm_rope_rows_kernel(
   }
 }
 
+// The plain case in one launch: columns q [H*D] | k [G*D] | v [G*V] of a
+// token's projection from `col`, rotate-half positions on the first rot_dims
+// dimensions of every q and k head, q densely in fp32, k and v to the token's
+// page rows. The token's cos and sin are evaluated once, for all heads. A
+// work item is a rotated pair or a single column.
+template <typename T>
+__global__ __launch_bounds__(BLOCK) void qkv_rope_rows_kernel(
+    const T* __restrict__ src, int ld, int col, int H, int G, int D, int V,
+    int rot_dims, const double* __restrict__ freqs,
+    const int* __restrict__ tok_seq, const int* __restrict__ tok_pos,
+    const int* __restrict__ table, int P, float* __restrict__ q,
+    T* __restrict__ kpool, T* __restrict__ vpool) {
+  extern __shared__ float cs[];      // [half][2]
+  const int t = blockIdx.x;
+  const int pos = tok_pos[t];
+  const int half = rot_dims / 2;
+  for (int i = threadIdx.x; i < half; i += BLOCK) {
+    const double ang = (double)pos * freqs[i];
+    cs[2 * i] = (float)cos(ang);
+    cs[2 * i + 1] = (float)sin(ang);
+  }
+  __syncthreads();
+  const T* row = src + (int64_t)t * ld + col;
+  const int64_t prow =
+      (int64_t)table[(int64_t)tok_seq[t] * P + pos / PAGE] * G * PAGE +
+      pos % PAGE;
+  const int iph = D - half;          // items per head
+  const int nqk = (H + G) * iph;
+  for (int e = threadIdx.x; e < nqk + G * V; e += BLOCK) {
+    if (e >= nqk) {
+      const int c = e - nqk, g = c / V;
+      vpool[(prow + (int64_t)g * PAGE) * V + (c - g * V)] =
+          row[(H + G) * D + c];
+      continue;
+    }
+    const int hd = e / iph, r = e - hd * iph;
+    const bool pair = r < half;
+    const int d0 = pair ? r : r + half;
+    float x = ldv<T>(row + hd * D + d0), y = 0.f;
+    if (pair) {
+      const float u = x, v = ldv<T>(row + hd * D + d0 + half);
+      x = u * cs[2 * r] - v * cs[2 * r + 1];
+      y = v * cs[2 * r] + u * cs[2 * r + 1];
+    }
+    if (hd < H) {
+      float* o = q + ((int64_t)t * H + hd) * D + d0;
+      o[0] = x;
+      if (pair) o[half] = y;
+    } else {
+      T* o = kpool + (prow + (int64_t)(hd - H) * PAGE) * D + d0;
+      stv<T>(o, x);
+      if (pair) stv<T>(o + half, y);
+    }
+  }
+}
+
 // -------------------------------------------------------------- attention
 // lanes that cover one value row of V columns with 16-byte loads: the
 // power of two at or above V / 8
@@ -508,6 +564,25 @@ void tl_norm_rope_rows(const void* src, int ld, int col, int n_heads,
                        (float*)out, (bf16*)pool, head_norm, interleaved,
                        rot_mult, (const bf16*)mix_src, mix_ld, mix_col,
                        (const float*)mix_lam, temp_coef, temp_every);
+}
+
+void tl_qkv_rope_rows(const void* src, int ld, int col, int H, int G, int D,
+                      int V, int rot_dims, const void* freqs,
+                      const void* tok_seq, const void* tok_pos,
+                      const void* table, int P, int T, void* q, void* kpool,
+                      void* vpool, int is_f32, hipStream_t stream) {
+  if (T <= 0) return;
+  dim3 grid(T), block(BLOCK);
+  const size_t smem = sizeof(float) * (size_t)rot_dims;
+#define TL_QR(TT)                                                           \
+  hipLaunchKernelGGL(qkv_rope_rows_kernel<TT>, grid, block, smem, stream,   \
+                     (const TT*)src, ld, col, H, G, D, V, rot_dims,         \
+                     (const double*)freqs, (const int*)tok_seq,             \
+                     (const int*)tok_pos, (const int*)table, P, (float*)q,  \
+                     (TT*)kpool, (TT*)vpool)
+  if (is_f32) TL_QR(float);
+  else TL_QR(bf16);
+#undef TL_QR
 }
 
 // heads per block for a shape: the largest of 8, 4, 2, 1 that divides the

@@ -24,8 +24,9 @@
 // and B[k][i] of one k per instruction and receives rows 4g .. 4g + 3 of
 // column i. The order of the k's is free: group g takes k = 4g + s at step s.
 // The scores are computed transposed (keys as rows), so their accumulator is
-// the A operand of the product with the values as it stands. Column n of a
-// value tile is column i * NV + n of memory: a lane's columns are contiguous.
+// the A operand of the product with the values as it stands. Column i of value
+// tile n is column 64 (n / 4) + 4 i + n % 4 of memory: a lane's columns come
+// in fours, and the fours of neighbouring lanes are contiguous.
 
 #include "common.hpp"
 
@@ -93,15 +94,17 @@ DEVINLINE void chunk_gates(const MlSrc& p, int t0, int n, int h, int H,
   a[t] = t < n ? li - f : -INFINITY;
 }
 
-// NV columns from c; columns beyond V (a multiple of 4) read as 0
+// a lane's NV columns from c; columns beyond V (a multiple of 4) read as 0. Loads are
+// unconditional, from the nearest place that exists: no branch around a load,
+// so that many are in flight together.
 template <int NV, typename T>
 DEVINLINE void ld_cols(const T* row, int c, int V, float (&o)[NV]) {
 #pragma unroll
   for (int n = 0; n < NV; n += 4) {
-    float x[4] = {0.f, 0.f, 0.f, 0.f};
-    if (c + n < V) ld4(row + c + n, x);
+    float x[4];
+    ld4(row + min(c + n * 16, V - 4), x);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) o[n + e] = x[e];
+    for (int e = 0; e < 4; ++e) o[n + e] = c + n * 16 < V ? x[e] : 0.f;
   }
 }
 
@@ -136,7 +139,7 @@ __global__ __launch_bounds__(BLOCK) void mlstm_state_kernel(
   const int nd = (D + 15) / 16, nv = (V + 16 * NV - 1) / (16 * NV);
   float* Uc = U + ci * D * V;
   for (int u = wave; u < nd * nv; u += 4) {
-    const int d0 = (u % nd) * 16, c = (u / nd) * 16 * NV + li * NV;
+    const int d0 = (u % nd) * 16, c = (u / nd) * 16 * NV + li * 4;
     f32x4 acc[NV];
 #pragma unroll
     for (int x = 0; x < NV; ++x) acc[x] = (f32x4){0.f, 0.f, 0.f, 0.f};
@@ -145,18 +148,14 @@ __global__ __launch_bounds__(BLOCK) void mlstm_state_kernel(
 #pragma unroll 4
     for (int s = 0; s < C / 4; ++s) {
       const int j = quad * (C / 4) + s;
-      float kw = 0.f, vv[NV];
-#pragma unroll
-      for (int x = 0; x < NV; ++x) vv[x] = 0.f;
-      if (j < n) {
-        const T* row = proj + (int64_t)(t0 + j) * p.ld;
-        if (din) {
-          if constexpr (sizeof(T) == 2) kw = bf2f(row[p.k_off + h * D + d0 + li]);
-          else kw = row[p.k_off + h * D + d0 + li];
-          kw *= w[j];
-        }
-        ld_cols<NV, T>(row + p.v_off + h * V, c, V, vv);
-      }
+      const T* row = proj + (int64_t)(t0 + min(j, n - 1)) * p.ld;
+      float kw, vv[NV];
+      if constexpr (sizeof(T) == 2)
+        kw = bf2f(row[p.k_off + h * D + min(d0 + li, D - 1)]);
+      else
+        kw = row[p.k_off + h * D + min(d0 + li, D - 1)];
+      kw = din ? kw * w[j] : 0.f;    // w is 0 beyond the chunk's tokens
+      ld_cols<NV, T>(row + p.v_off + h * V, c, V, vv);
       ns += kw;
 #pragma unroll
       for (int x = 0; x < NV; ++x)
@@ -169,10 +168,10 @@ __global__ __launch_bounds__(BLOCK) void mlstm_state_kernel(
       if (d >= D) continue;
 #pragma unroll
       for (int x = 0; x < NV; x += 4)
-        if (c + x < V) {
+        if (c + x * 16 < V) {
           const float o[4] = {acc[x][r], acc[x + 1][r], acc[x + 2][r],
                               acc[x + 3][r]};
-          st4(Uc + (int64_t)d * V + c + x, o);
+          st4(Uc + (int64_t)d * V + c + x * 16, o);
         }
     }
     if (u < nd) {                    // the same with v = 1
@@ -302,7 +301,7 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
   const int li = lane & 15, quad = lane >> 4;
   if (wave * 16 >= n) return;        // no barrier below
   const int t = wave * 16 + li;      // this lane's query
-  const int c = li * NV;             // and its first value column
+  const int c = li * 4;              // and its first value column
   const T* kh = proj + (int64_t)t0 * p.ld + p.k_off + h * D;
   const T* vh = proj + (int64_t)t0 * p.ld + p.v_off + h * V;
   const double Mt = M[t];
@@ -312,16 +311,13 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
   const float* n0 = nU + ci * D;
 #pragma unroll
   for (int dt = 0; dt < DT; ++dt) {
-    const int d = dt * 16 + quad * 4;
-    float x[4] = {0.f, 0.f, 0.f, 0.f}, y[4] = {0.f, 0.f, 0.f, 0.f};
-    if (d < D) {
-      if (t < n)
-        ld4(proj + (int64_t)(t0 + t) * p.ld + p.q_off + h * D + d, x);
-      ld4(n0 + d, y);
-    }
+    const int d = dt * 16 + quad * 4, dc = min(d, D - 4);
+    float x[4], y[4];
+    ld4(proj + (int64_t)(t0 + min(t, n - 1)) * p.ld + p.q_off + h * D + dc, x);
+    ld4(n0 + dc, y);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      q[dt][e] = x[e] * p.qscale;
+      q[dt][e] = d < D && t < n ? x[e] * p.qscale : 0.f;
       nq += q[dt][e] * y[e];
     }
   }
@@ -337,10 +333,8 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int d = dt * 16 + quad * 4 + e;
-        float s0[NV];
-#pragma unroll
-        for (int x = 0; x < NV; ++x) s0[x] = 0.f;
-        if (d < D) ld_cols<NV, float>(Uc + (int64_t)d * V, c, V, s0);
+        float s0[NV];                // (q is 0 beyond D)
+        ld_cols<NV, float>(Uc + (int64_t)min(d, D - 1) * V, c, V, s0);
         const float qe = q[dt][e] * carry;
 #pragma unroll
         for (int x = 0; x < NV; ++x)
@@ -355,9 +349,9 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
     const int j = b * 16 + li;       // this lane's key row
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      const int d = dt * 16 + quad * 4;
-      float x[4] = {0.f, 0.f, 0.f, 0.f};
-      if (d < D && j < n) ld4(kh + (int64_t)j * p.ld + d, x);
+      float x[4];                    // (q is 0 beyond D, rows beyond n masked)
+      ld4(kh + (int64_t)min(j, n - 1) * p.ld +
+              min(dt * 16 + quad * 4, D - 4), x);
 #pragma unroll
       for (int e = 0; e < 4; ++e)
         sc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[e], q[dt][e], sc, 0, 0, 0);
@@ -368,9 +362,7 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
       const float w = s <= t && s < n ? sc[e] * expf((float)(a[s] - Mt)) : 0.f;
       nq += w;
       float vv[NV];
-#pragma unroll
-      for (int x = 0; x < NV; ++x) vv[x] = 0.f;
-      if (s < n) ld_cols<NV, T>(vh + (int64_t)s * p.ld, c, V, vv);
+      ld_cols<NV, T>(vh + (int64_t)min(s, n - 1) * p.ld, c, V, vv);
 #pragma unroll
       for (int x = 0; x < NV; ++x)
         acc[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(w, vv[x], acc[x], 0, 0,
@@ -402,14 +394,14 @@ __global__ __launch_bounds__(BLOCK) void mlstm_out_kernel(
       T* orow = out + (row * H + h) * V;
 #pragma unroll
       for (int x = 0; x < NV; x += 4)
-        if (c + x < V) {
+        if (c + x * 16 < V) {
           float g[4], w4[4], o[4];
-          ld4(gr + c + x, g);
-          ld4(norm_w + h * V + c + x, w4);
+          ld4(gr + c + x * 16, g);
+          ld4(norm_w + h * V + c + x * 16, w4);
 #pragma unroll
           for (int e = 0; e < 4; ++e)
             o[e] = acc[x + e][r] * rn * w4[e] / (1.f + expf(-g[e]));
-          st4(orow + c + x, o);
+          st4(orow + c + x * 16, o);
         }
     }
   }

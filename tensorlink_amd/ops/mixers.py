@@ -660,6 +660,24 @@ def norm_rope_rows(src: torch.Tensor, col: int, n_heads: int, head_dim: int,
     return None
 
 
+def qkv_rope_rows(src: torch.Tensor, col: int, H: int, rot_dims: int,
+                  freqs: Optional[torch.Tensor], meta: RaggedMeta,
+                  kpool: torch.Tensor, vpool: torch.Tensor) -> torch.Tensor:
+    """Row preparation of plain rotated attention in one launch: columns
+    q [H*D] | k [G*D] | v [G*V] of src from ``col``; rotate-half positions
+    on the first ``rot_dims`` dimensions of every q and k head; k and v go
+    to the tokens' page rows, q is returned densely, fp32 [T, H*D]."""
+    G, D, V = kpool.shape[1], kpool.shape[3], vpool.shape[3]
+    if src.is_cuda:
+        return _ext().qkv_rope_rows(src, int(col), int(H), int(rot_dims),
+                                    freqs, meta.tok_seq, meta.tok_pos,
+                                    meta.table, kpool, vpool)
+    rot = dict(rot_dims=rot_dims, freqs=freqs)
+    norm_rope_rows(src, col + H * D, G, D, meta, pool=kpool, **rot)
+    norm_rope_rows(src, col + (H + G) * D, G, V, meta, pool=vpool)
+    return norm_rope_rows(src, col, H, D, meta, **rot)
+
+
 # ---------------------------------------------------------------------------
 # softmax attention over the paged pool with the options layered models
 # combine: GQA/MQA, sliding window, sink, cross-head score mixing, values
@@ -1292,12 +1310,6 @@ def expert_gated_ff(h: torch.Tensor, wts: torch.Tensor, idx: torch.Tensor,
 # ---------------------------------------------------------------------------
 # gated delta rule, bigram embedding, thin fp32 projections
 # ---------------------------------------------------------------------------
-def delta_chunk(D: int) -> int:
-    """Tokens per chunk of the chunk form of the gated delta rule for key
-    size D; 0 if the chunk kernels do not serve it."""
-    return 64 if D <= 64 else 32 if D <= 256 else 0
-
-
 def delta_scan(x: torch.Tensor, offs, proj: torch.Tensor, r_off: int,
                b: torch.Tensor, b_off: int, a2t: torch.Tensor,
                dt_bias: torch.Tensor, A_log: torch.Tensor, S: torch.Tensor,
@@ -1320,19 +1332,19 @@ def delta_scan(x: torch.Tensor, offs, proj: torch.Tensor, r_off: int,
     assert x.dtype == b.dtype == S.dtype == torch.float32
     assert a2t.dtype == dt_bias.dtype == A_log.dtype == torch.float32
     if x.is_cuda:
-        C = delta_chunk(D)
         args = (x, q_off, k_off, v_off, proj, int(r_off), b, int(b_off), a2t,
                 dt_bias, A_log, S)
-        if (C and max(meta.new_h) >= 2 * C
+        C = _ext().delta_chunk_tokens()
+        if (max(meta.new_h) >= 2 * C
                 and not os.environ.get("TL_NO_SCAN_CHUNKS")
                 and T * H * (3 * D + C + V) * 4 <= (1 << 33)
-                and _ext().delta_chunks_ok(int(D), int(R), C)):
+                and _ext().delta_chunks_ok(int(D), int(R))):
             # long prompt portions: per-chunk factors in parallel, then the
             # chain over a sequence's chunks
             cu_c, _, _, base, cnt, nc, _ = meta.scan_chunks(C)
             return _ext().delta_chunks(*args, cu_c, base, cnt, meta.slots,
                                        meta.pos0, int(H), int(G), int(D),
-                                       int(V), int(C))
+                                       int(V))
         return _ext().delta_scan(*args, meta.cu, meta.slots, meta.pos0,
                                  int(H), int(G), int(D), int(V))
     F = torch.nn.functional
