@@ -631,6 +631,102 @@ def test_delta_state_across_a_batch(device, dtype, H, G, D, V):
         assert torch.equal(S[2].cpu(), S0[2])
 
 
+@pytest.mark.parametrize("H,D,V", [(3, 20, 12), (2, 64, 80), (1, 100, 132),
+                                   (2, 7, 9)])
+@pytest.mark.parametrize("device,dtype", ALL)
+def test_mlstm_state_across_a_batch(device, dtype, H, D, V):
+    """The op on a ragged batch of fresh and continued sequences in
+    shuffled slots, chunk forms and token walk: outputs and the states
+    left behind equal each sequence alone; untouched slots stay."""
+    g = torch.Generator().manual_seed(9)
+    new, pos0, slots = [150, 1, 257, 2], [0, 70, 5, 0], [4, 0, 3, 1]
+    T, cap, eps = sum(new), 15.0, 1e-5
+    offs = (0, H * D, 2 * H * D, 2 * H * D + H * V)
+    proj = torch.randn(T, offs[3] + H * V + (4 if D % 4 == 0 else 3),
+                       generator=g).to(dtype)
+    gates = torch.randn(T, 2 * H + 3, generator=g) * 3
+    nw = 1.0 + 0.2 * torch.randn(H * V, generator=g)
+    S0 = torch.randn(5, H, D, V, generator=g)
+    n0, m0 = torch.randn(5, H, D, generator=g), torch.rand(5, H, generator=g)
+    f, gt = proj.double().numpy(), gates.double().numpy()
+    want, states, at = np.zeros((T, H, V)), {}, 0
+    for cnt, p, s in zip(new, pos0, slots):
+        S, n, m = (x[s].double().numpy().copy() * (p > 0)
+                   for x in (S0, n0, m0))
+        for t in range(at, at + cnt):
+            for h in range(H):
+                q, k, v, _ = (f[t, o + h * w:o + (h + 1) * w]
+                              for o, w in zip(offs, (D, D, V, V)))
+                li = cap * math.tanh(gt[t, h] / cap)
+                lf = -O.softplus(-cap * math.tanh(gt[t, H + h] / cap))
+                top = max(lf + m[h], li)
+                a, b = math.exp(lf + m[h] - top), math.exp(li - top)
+                S[h] = a * S[h] + b * np.outer(k, v)
+                n[h] = a * n[h] + b * k
+                m[h] = top
+                q = q / math.sqrt(D)
+                want[t, h] = (S[h].T @ q) / (
+                    max(abs(n[h] @ q), math.exp(-top)) + 1e-6)
+        states[s] = (S, n, m)
+        at += cnt
+    want = O.rms(want, eps).reshape(T, H * V) * nw.double().numpy() \
+        * O.sigmoid(f[:, offs[3]:offs[3] + H * V])
+    meta = mx.RaggedMeta(new, pos0, slots, torch.zeros(4, 2,
+                         dtype=torch.int32).to(device), device)
+    lim = 2e-4 if dtype == torch.float32 else 2e-2
+    for chunks in (True, False):
+        if not chunks:
+            os.environ["TL_NO_SCAN_CHUNKS"] = "1"
+        try:
+            S, n, m = (x.to(device).clone() for x in (S0, n0, m0))
+            got = mx.mlstm_scan(proj.to(device), offs, gates.to(device),
+                                nw.to(device), S, n, m, meta, H, D, V, cap,
+                                eps)
+        finally:
+            os.environ.pop("TL_NO_SCAN_CHUNKS", None)
+        # a normaliser near zero makes single rows ill-conditioned
+        err = np.abs(got.float().cpu().numpy() - want).max(-1)
+        assert np.quantile(err, 0.98) < lim * np.abs(want).max()
+        for s, st in states.items():
+            for x, y in zip((S, n, m), st):
+                assert np.abs(x[s].cpu().numpy() - y).max() < \
+                    1e-4 * np.abs(y).max()
+        assert torch.equal(S[2].cpu(), S0[2])
+        assert torch.equal(m[2].cpu(), m0[2])
+
+
+@pytest.mark.parametrize("device,dtype", ALL)
+def test_short_convolution(device, dtype):
+    """The convolution with silu on a ragged batch, one to nine taps, with
+    and without the vector path: portions shorter and longer than the taps,
+    slots that hold another sequence's inputs before the first step."""
+    g = torch.Generator().manual_seed(8)
+    for N, K, col in ((12, 1, 4), (8, 2, 0), (16, 4, 8), (2052, 4, 4),
+                      (12, 9, 4), (7, 3, 1), (10, 5, 2), (12, 6, 8)):
+        seqs = [torch.randn(n, N + col + 4, generator=g).to(dtype)
+                for n in (40, 3, 17)]
+        taps = torch.randn(N, K, generator=g)
+        want = [O.short_conv_silu(s[:, col:col + N].double().numpy(),
+                                  taps.double().numpy()) for s in seqs]
+        hist = torch.randn(5, K - 1, N, generator=g).to(device)
+        slots, at = [3, 0, 4], [0, 0, 0]
+        for step in ([9, 1, 2], [1, 1, 1], [30, 0, 14], [0, 1, 0]):
+            live = [i for i in range(3) if step[i]]
+            meta = mx.RaggedMeta(
+                [step[i] for i in live], [at[i] for i in live],
+                [slots[i] for i in live],
+                torch.zeros(len(live), 1, dtype=torch.int32).to(device),
+                device)
+            src = torch.cat([seqs[i][at[i]:at[i] + step[i]] for i in live])
+            got = mx.conv_rope_rows(src.to(device), col, 1, N,
+                                    taps.to(device), hist, meta, silu=True)
+            ref = np.concatenate([want[i][at[i]:at[i] + step[i]]
+                                  for i in live])
+            assert np.abs(got.cpu().numpy() - ref).max() < 2e-5, (N, K)
+            for i in live:
+                at[i] += step[i]
+
+
 @pytest.mark.parametrize("hgdv,rot,size", [
     ((4, 2, 12, 10), 6, 21), ((1, 1, 16, 16), 16, 1),
     ((8, 2, 24, 136), 8, 100), ((4, 2, 24, 48), 24, 64),
